@@ -91,3 +91,12 @@ def _zasidra() -> None:
 
 
 _zasidra()
+
+
+def _peponex() -> None:
+    from ..models.peponex import peponex_spec
+    from .peponex_config import PeponexConfig
+    register_architecture("Peponex", PeponexConfig.from_dict, peponex_spec, reads_shapes=True)
+
+
+_peponex()

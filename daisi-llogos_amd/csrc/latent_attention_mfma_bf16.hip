@@ -3,7 +3,8 @@
 // [latent | rotated part | zeros] of `row` dimensions (a multiple of 16) in the key pool; the
 // values are the latent again, in a value pool of the same page shape, in the matrix cores'
 // operand order for O^T += V^T . P^T (common.h).  Softmax state and sums are 32-bit; a head's
-// learned sink joins the denominator once.
+// learned sink joins the denominator once.  With a window a query sees the last `window` keys, its own
+// among them; pages before the first that a tile's first query can see are not touched.
 //
 // Work: the (token, head) pairs of a sequence's part of the step, token-major, in tiles of 16
 // columns; a wave owns one tile, with its queries as second operands in registers, and takes
@@ -57,7 +58,7 @@ __global__ __launch_bounds__(kLatentWaves* kWave) void latent_attn_kernel(
         bf16_t* __restrict__ out, int dv, const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pool,
         const bf16_t* __restrict__ v_pool, const int* __restrict__ table, int table_stride,
         const int* __restrict__ cu, const int* __restrict__ tok_pos, int batch, int n_heads, int row,
-        float scale, const float* __restrict__ head_sink, int splits, int pages_per_split,
+        float scale, int window, const float* __restrict__ head_sink, int splits, int pages_per_split,
         float* __restrict__ ws_ml, float* __restrict__ ws_acc, int total_cols, int n_tiles) {
     const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
     const int c = lane & 15, g = lane >> 4;
@@ -89,7 +90,8 @@ __global__ __launch_bounds__(kLatentWaves* kWave) void latent_attn_kernel(
     const int pos_hi = tok_pos[first_tok + last_col / n_heads], pos_lo = tok_pos[first_tok + (tile_in_seq * 16) / n_heads];
     const int n_pages = pos_hi / kPageTokens + 1;
     const int split = blockIdx.y;
-    const int page0 = split * pages_per_split, page1 = min(n_pages, page0 + pages_per_split);
+    const int seen_from = window > 0 ? max(0, pos_lo - window + 1) / kPageTokens : 0;        // the first page with a visible key
+    const int page0 = seen_from + split * pages_per_split, page1 = min(n_pages, page0 + pages_per_split);
 
     const int ksteps = (row + 31) / 32, dvt = (dv + 15) / 16, octs = row >> 3;
     lbf16x8 qf[KS];
@@ -127,13 +129,15 @@ __global__ __launch_bounds__(kLatentWaves* kWave) void latent_attn_kernel(
             }
         }
         // softmax of the page: this lane holds, for its column, keys key0 + 16 g + 4 rb + r
-        const bool masked = key0 + kPageTokens - 1 > pos_lo;
+        const bool masked = key0 + kPageTokens - 1 > pos_lo || (window > 0 && key0 <= pos_hi - window);
+        const int q_from = window > 0 ? q_pos - window + 1 : 0;                              // this column's first visible key
         float tile_max = -INFINITY;
 #pragma unroll
         for (int rb = 0; rb < 4; ++rb)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                if (masked && key0 + 16 * g + 4 * rb + r > q_pos) s[rb][r] = -INFINITY;
+                const int key = key0 + 16 * g + 4 * rb + r;
+                if (masked && (key > q_pos || key < q_from)) s[rb][r] = -INFINITY;
                 tile_max = fmaxf(tile_max, s[rb][r]);
             }
         tile_max = col_max(tile_max);
@@ -263,11 +267,11 @@ LLOGOS_EXPORT long long llogos_latent_attn_workspace(int total_cols, int dv, int
 // ceil(tokens * heads / 16).  Returns LLOGOS_UNSUPPORTED for rows of more than 576 dimensions.
 LLOGOS_EXPORT int llogos_latent_attn_bf16(void* out, int dv, const void* q, const void* k_pool, const void* v_pool,
                                           const int* table, int table_stride, const int* cu, const int* tok_pos,
-                                          int batch, int T, int n_heads, int row, float scale, const float* head_sink,
+                                          int batch, int T, int n_heads, int row, float scale, int window, const float* head_sink,
                                           int n_tiles, int splits, int pages_per_split, float* workspace,
                                           long long workspace_floats, hipStream_t stream) {
     if (T <= 0 || batch <= 0 || n_heads <= 0 || row <= 0 || row % 16 || dv <= 0 || dv > row || n_tiles <= 0) return LLOGOS_BAD_ARGUMENT;
-    if (splits < 1 || splits > kMergeSplits || pages_per_split < 1 || (!cu && T != batch)) return LLOGOS_BAD_ARGUMENT;
+    if (splits < 1 || splits > kMergeSplits || pages_per_split < 1 || window < 0 || (!cu && T != batch)) return LLOGOS_BAD_ARGUMENT;
     if (row > 576) return LLOGOS_UNSUPPORTED;
     const int total_cols = T * n_heads, dvp = (dv + 15) / 16 * 16;
     float *ws_ml = nullptr, *ws_acc = nullptr;
@@ -278,7 +282,7 @@ LLOGOS_EXPORT int llogos_latent_attn_bf16(void* out, int dv, const void* q, cons
     }
     dim3 grid((n_tiles + kLatentWaves - 1) / kLatentWaves, splits);
 #define LAT(KS, DVT) latent_attn_kernel<KS, DVT><<<grid, kLatentWaves * kWave, 0, stream>>>((bf16_t*)out, dv, (const bf16_t*)q, \
-        (const bf16_t*)k_pool, (const bf16_t*)v_pool, table, table_stride, cu, tok_pos, batch, n_heads, row, scale, head_sink, \
+        (const bf16_t*)k_pool, (const bf16_t*)v_pool, table, table_stride, cu, tok_pos, batch, n_heads, row, scale, window, head_sink, \
         splits, pages_per_split, ws_ml, ws_acc, total_cols, n_tiles)
     if (row <= 128) LAT(4, 8);
     else if (row <= 256) LAT(8, 16);

@@ -65,6 +65,8 @@ __device__ __forceinline__ float moe_gated(float gate, float up) { return gate /
 // out[r, :] = act(a_row(r) . w[e]^T) * scale for the sorted rows r of expert e's segment.
 // act 0: none; 1: the square of relu; 2: the matrix's rows are gate and up rows in turn (gate 0, up 0, gate 1, ...)
 // and the result has N / 2 columns silu(gate_i) * up_i.
+// With row_weight (act 2 only) a row's gate and up sums are multiplied by row_weight[order[r]] first: the product of the
+// row times its pair's weight.
 // a_row(r) = a[order[r] / top] when gather (the step's token rows), else a[r] (rows already sorted).
 // w is [E][N][K].  Tiles of 64 rows x 64 columns; blockIdx.y counts row tiles over all segments.
 constexpr int GM = 64, GN = 64, GK = 16;
@@ -72,7 +74,8 @@ constexpr int GM = 64, GN = 64, GK = 16;
 template <typename TA, typename TW, typename TO>
 __global__ __launch_bounds__(256) void moe_product_kernel(TO* __restrict__ out, const TA* __restrict__ a, const TW* __restrict__ w,
                                                           const int* __restrict__ order, const int* __restrict__ seg, int E,
-                                                          int top, int gather, int N, int K, int lda, int act, float scale) {
+                                                          int top, int gather, int N, int K, int lda, int act, float scale,
+                                                          const float* __restrict__ row_weight) {
     __shared__ float As[GK][GM + 4];
     __shared__ float Ws[GK][GN + 4];
     __shared__ int src_row[GM];
@@ -136,13 +139,14 @@ __global__ __launch_bounds__(256) void moe_product_kernel(TO* __restrict__ out, 
     for (int i = 0; i < 4; ++i) {
         const int m = m0 + ty * 4 + i;
         if (m >= m_end) continue;
+        const float rw = row_weight ? row_weight[order[m]] : 1.0f;
         if (act == 2) {                                     // columns in pairs (gate, up): silu(gate) * up
 #pragma unroll
             for (int j = 0; j < 4; j += 2) {
                 const int n = n0 + tx * 4 + j;
                 if (n + 1 >= N) continue;
                 const float gt = acc[i][j] + mid[i][j], up = acc[i][j + 1] + mid[i][j + 1];
-                store_f32(out + (size_t)m * (N / 2) + n / 2, moe_gated(gt, up) * scale);
+                store_f32(out + (size_t)m * (N / 2) + n / 2, moe_gated(gt * rw, up * rw) * scale);
             }
             continue;
         }
@@ -160,13 +164,13 @@ __global__ __launch_bounds__(256) void moe_product_kernel(TO* __restrict__ out, 
 // P = T * top sorted rows at most; row_tiles bounds the tiles of all segments: ceil(P / 64) + E covers them.
 LLOGOS_EXPORT int llogos_moe_product(void* out, int out_dtype, const void* a, int a_dtype, const void* w, int w_dtype,
                                      const int* order, const int* seg, int E, int top, int gather, int P, int N, int K,
-                                     int lda, int act, float scale, hipStream_t stream) {
-    if (P <= 0 || N <= 0 || K <= 0 || E <= 0 || top <= 0 || lda < K || act < 0 || act > 2 || (act == 2 && (N & 1))) return LLOGOS_BAD_ARGUMENT;
+                                     int lda, int act, float scale, const float* row_weight, hipStream_t stream) {
+    if (P <= 0 || N <= 0 || K <= 0 || E <= 0 || top <= 0 || lda < K || act < 0 || act > 2 || (act == 2 && (N & 1)) || (row_weight && act != 2)) return LLOGOS_BAD_ARGUMENT;
     if (a_dtype != w_dtype && !(a_dtype == DT_F32)) return LLOGOS_BAD_ARGUMENT;
     const int row_tiles = (P + GM - 1) / GM + E;
     dim3 grid((N + GN - 1) / GN, row_tiles);
 #define MP(TA, TW, TO) moe_product_kernel<TA, TW, TO><<<grid, 256, 0, stream>>>((TO*)out, (const TA*)a, (const TW*)w, order, seg, E, \
-        top, gather, N, K, lda, act, scale)
+        top, gather, N, K, lda, act, scale, row_weight)
     if (a_dtype == DT_F32 && w_dtype == DT_F32 && out_dtype == DT_F32) MP(float, float, float);
     else if (a_dtype == DT_BF16 && w_dtype == DT_BF16 && out_dtype == DT_BF16) MP(bf16_t, bf16_t, bf16_t);
     else if (a_dtype == DT_BF16 && w_dtype == DT_BF16 && out_dtype == DT_F32) MP(bf16_t, bf16_t, float);
@@ -323,9 +327,10 @@ __device__ __forceinline__ int wave_best_open(const float* v, const unsigned cha
 //   `keep` best groups cannot be chosen (n_groups <= 1 or keep >= n_groups: all can)
 //   choice[t, j] = the j-th largest c that can be chosen (the lowest index among equals), j < top
 //   weight[t, j] = s[choice] / (sum_j s[choice_j] + 1e-20) * scale
+// With `sigmoid` s is the logistic function of every logit by itself; without `renorm` the weights are s[choice] * scale.
 // The caller sees to it that the kept groups hold at least `top` outputs.
 __global__ __launch_bounds__(kWave) void moe_router_choose_kernel(const float* __restrict__ z, const float* __restrict__ correction,
-                                                                  int E, int n_groups, int keep, int top, float scale,
+                                                                  int E, int n_groups, int keep, int top, float scale, int sigmoid, int renorm,
                                                                   int* __restrict__ choice, float* __restrict__ weight) {
     __shared__ float s[kMoeMaxExperts], c[kMoeMaxExperts], gbest[kMoeMaxExperts], picked_s[kMoeMaxExperts];
     __shared__ int picked[kMoeMaxExperts];
@@ -336,8 +341,12 @@ __global__ __launch_bounds__(kWave) void moe_router_choose_kernel(const float* _
     for (int e = lane; e < E; e += kWave) { const float v = zr[e]; s[e] = v; m = fmaxf(m, v); }
     m = wave_max(m);
     float sum = 0.f;
-    for (int e = lane; e < E; e += kWave) { const float v = expf(s[e] - m); s[e] = v; sum += v; }
-    sum = wave_sum(sum);
+    for (int e = lane; e < E; e += kWave) {
+        const float v = sigmoid ? 1.0f / (1.0f + expf(-s[e])) : expf(s[e] - m);
+        s[e] = v;
+        sum += v;
+    }
+    sum = sigmoid ? 1.0f : wave_sum(sum);
     for (int e = lane; e < E; e += kWave) {
         const float v = s[e] / sum;
         s[e] = v;
@@ -371,7 +380,7 @@ __global__ __launch_bounds__(kWave) void moe_router_choose_kernel(const float* _
         __syncthreads();
         total += s[e];
     }
-    const float f = scale / (total + 1e-20f);
+    const float f = renorm ? scale / (total + 1e-20f) : scale;
     for (int j = lane; j < top; j += kWave) {
         choice[(size_t)t * top + j] = picked[j];
         weight[(size_t)t * top + j] = picked_s[j] * f;
@@ -379,50 +388,53 @@ __global__ __launch_bounds__(kWave) void moe_router_choose_kernel(const float* _
 }
 
 LLOGOS_EXPORT int llogos_moe_router_choose(const float* z, const float* correction, int T, int E, int n_groups, int keep, int top,
-                                           float scale, int* choice, float* weight, hipStream_t stream) {
+                                           float scale, int sigmoid, int renorm, int* choice, float* weight, hipStream_t stream) {
     if (T <= 0 || E <= 0 || E > kMoeMaxExperts || top <= 0 || top > E) return LLOGOS_BAD_ARGUMENT;
     if (n_groups > 1 && (E % n_groups || keep < 1 || (long long)min(keep, n_groups) * (E / n_groups) < top)) return LLOGOS_BAD_ARGUMENT;
-    moe_router_choose_kernel<<<T, kWave, 0, stream>>>(z, correction, E, n_groups, keep, top, scale, choice, weight);
+    moe_router_choose_kernel<<<T, kWave, 0, stream>>>(z, correction, E, n_groups, keep, top, scale, sigmoid, renorm, choice, weight);
     return LLOGOS_LAUNCH_CHECK();
 }
 
 // out[t, :] = sum_j weight[t, j] * row_j + (sum of the parts of shared[t, :]), with row_j = y[where[t * top + j], :] when
 // choice[t, j] < n_real and the token's own row a[t, :] otherwise (a router output without matrices returns its input).
-// y float32 [P, W]; a [T, lda] of any storage type; shared float32 [(parts,) T, W] or null.
+// y float32 [P, W]; a [T, lda] of any storage type; shared float32 [(parts,) T, W] or null.  weight null: every row counts
+// once.  `add`: the result joins what out holds (the float32 stream), and with `rows` the new rows are left in that type too.
 template <typename TA>
 __global__ void moe_combine_weighted_kernel(float* __restrict__ out, const float* __restrict__ y, const int* __restrict__ where,
                                             const int* __restrict__ choice, const float* __restrict__ weight, int top, int n_real,
                                             const TA* __restrict__ a, int lda, const float* __restrict__ shared_rows, int parts,
-                                            size_t part_stride, int T, int W) {
+                                            size_t part_stride, int T, int W, int add, TA* __restrict__ rows) {
     const int t = blockIdx.x;
     for (int col = blockIdx.y * blockDim.x + threadIdx.x; col < W; col += gridDim.y * blockDim.x) {
         float v = 0.f;
         for (int j = 0; j < top; ++j) {
             const int p = t * top + j;
             const float row = choice[p] < n_real ? y[(size_t)where[p] * W + col] : load_f32(a + (size_t)t * lda + col);
-            v = fmaf(weight[p], row, v);
+            v = weight ? fmaf(weight[p], row, v) : v + row;
         }
         if (shared_rows) {
             float sh = shared_rows[(size_t)t * W + col];
             for (int q = 1; q < parts; ++q) sh += shared_rows[q * part_stride + (size_t)t * W + col];
             v += sh;
         }
+        if (add) v += out[(size_t)t * W + col];
+        if (rows) store_f32(rows + (size_t)t * W + col, v);
         out[(size_t)t * W + col] = v;
     }
 }
 
 LLOGOS_EXPORT int llogos_moe_combine_weighted(float* out, const float* y, const int* where, const int* choice, const float* weight,
                                               int top, int n_real, const void* a, int a_dtype, int lda, const float* shared_rows,
-                                              int parts, long long part_stride, int T, int W, hipStream_t stream) {
+                                              int parts, long long part_stride, int T, int W, int add, void* rows, hipStream_t stream) {
     if (T <= 0 || W <= 0 || top <= 0 || parts < 1 || lda < W || n_real < 0) return LLOGOS_BAD_ARGUMENT;
     const int threads = 256;
     dim3 grid(T, (W + threads - 1) / threads);
     if (a_dtype == DT_F32)
         moe_combine_weighted_kernel<float><<<grid, threads, 0, stream>>>(out, y, where, choice, weight, top, n_real, (const float*)a, lda,
-                                                                         shared_rows, parts, (size_t)part_stride, T, W);
+                                                                         shared_rows, parts, (size_t)part_stride, T, W, add, (float*)rows);
     else if (a_dtype == DT_BF16)
         moe_combine_weighted_kernel<bf16_t><<<grid, threads, 0, stream>>>(out, y, where, choice, weight, top, n_real, (const bf16_t*)a, lda,
-                                                                          shared_rows, parts, (size_t)part_stride, T, W);
+                                                                          shared_rows, parts, (size_t)part_stride, T, W, add, (bf16_t*)rows);
     else return LLOGOS_BAD_ARGUMENT;
     return LLOGOS_LAUNCH_CHECK();
 }
@@ -475,7 +487,8 @@ __device__ __forceinline__ void moe_find_tile(const int* __restrict__ seg, int E
 template <typename TO>
 __global__ __launch_bounds__(256) void moe_few_kernel(TO* __restrict__ out, const bf16_t* __restrict__ a, const bf16_t* __restrict__ w,
                                                       const int* __restrict__ order, const int* __restrict__ seg, int E, int top,
-                                                      int gather, int N, int K, int lda, int act, float scale) {
+                                                      int gather, int N, int K, int lda, int act, float scale,
+                                                      const float* __restrict__ row_weight) {
     __shared__ float red[3][kWave][4];
     __shared__ int s_tile[3];
     if (threadIdx.x == 0) moe_find_tile(seg, E, 16, blockIdx.y, s_tile[0], s_tile[1], s_tile[2]);
@@ -513,8 +526,10 @@ __global__ __launch_bounds__(256) void moe_few_kernel(TO* __restrict__ out, cons
     }
     const int n = n0 + 4 * g;
     if (m < m_end && n < N) {
-        if (act == 2) moe_store2(out + (size_t)m * (N / 2) + n / 2, moe_gated(v[0], v[1]) * scale, moe_gated(v[2], v[3]) * scale);
-        else moe_store4(out + (size_t)m * N + n, v[0], v[1], v[2], v[3]);
+        if (act == 2) {
+            const float rw = row_weight ? row_weight[order[m]] : 1.0f;
+            moe_store2(out + (size_t)m * (N / 2) + n / 2, moe_gated(v[0] * rw, v[1] * rw) * scale, moe_gated(v[2] * rw, v[3] * rw) * scale);
+        } else moe_store4(out + (size_t)m * N + n, v[0], v[1], v[2], v[3]);
     }
 }
 
@@ -531,7 +546,8 @@ __device__ __forceinline__ int moe_lds_at(int row, int oct) { return row * kMoeB
 template <int BM, int BN, typename TO>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3, 3))) void moe_tiles_kernel(
         TO* __restrict__ out, const bf16_t* __restrict__ a, const bf16_t* __restrict__ w, const int* __restrict__ order,
-        const int* __restrict__ seg, int E, int top, int gather, int N, int K, int lda, int act, float scale) {
+        const int* __restrict__ seg, int E, int top, int gather, int N, int K, int lda, int act, float scale,
+                                                          const float* __restrict__ row_weight) {
     constexpr int CA = BM * 8 / 256, CW = BN * 8 / 256;           // 16-byte pieces a thread copies a stage
     constexpr int WN = BM == 128 ? BN / 2 : BN / 4, NT = WN / 32, MT = 2;     // a wave's part: 64 rows x WN columns of the tile
     __shared__ __attribute__((aligned(16))) bf16_t As[BM * kMoeBK];
@@ -615,6 +631,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3, 3))) voi
     for (int mt = 0; mt < MT; ++mt) {
         const int m = m0 + wm * 64 + mt * 32 + r32;
         if (m >= m_end) continue;
+        const float rw = row_weight ? row_weight[order[m]] : 1.0f;
 #pragma unroll
         for (int nt = 0; nt < NT; ++nt)
 #pragma unroll
@@ -628,7 +645,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3, 3))) voi
                     if (act == 1) { v[r] = fmaxf(v[r], 0.f); v[r] *= v[r]; }
                     if (act != 2) v[r] *= scale;
                 }
-                if (act == 2) moe_store2(out + (size_t)m * (N / 2) + n / 2, moe_gated(v[0], v[1]) * scale, moe_gated(v[2], v[3]) * scale);
+                if (act == 2) moe_store2(out + (size_t)m * (N / 2) + n / 2, moe_gated(v[0] * rw, v[1] * rw) * scale, moe_gated(v[2] * rw, v[3] * rw) * scale);
                 else moe_store4(out + (size_t)m * N + n, v[0], v[1], v[2], v[3]);
             }
     }
@@ -636,15 +653,15 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3, 3))) voi
 
 // form 0: few rows (tiles of 16); 1: tiles of 64 rows; 2: tiles of 128 rows.  -2 for shapes these do not take.
 LLOGOS_EXPORT int llogos_moe_product_bf16(void* out, int out_dtype, const void* a, const void* w, const int* order, const int* seg,
-                                          int E, int top, int gather, int P, int N, int K, int lda, int act, float scale, int form,
-                                          hipStream_t stream) {
-    if (P <= 0 || N <= 0 || K <= 0 || E <= 0 || top <= 0 || lda < K || act < 0 || act > 2 || form < 0 || form > 2) return LLOGOS_BAD_ARGUMENT;
+                                          int E, int top, int gather, int P, int N, int K, int lda, int act, float scale,
+                                          const float* row_weight, int form, hipStream_t stream) {
+    if (P <= 0 || N <= 0 || K <= 0 || E <= 0 || top <= 0 || lda < K || act < 0 || act > 2 || form < 0 || form > 2 || (row_weight && act != 2)) return LLOGOS_BAD_ARGUMENT;
     if ((K % 8) || (N % 4) || (lda % 8) || ((uintptr_t)a % 16) || ((uintptr_t)w % 16) || ((uintptr_t)out % 16)) return LLOGOS_UNSUPPORTED;
     if (out_dtype != DT_F32 && out_dtype != DT_BF16) return LLOGOS_BAD_ARGUMENT;
     const int rows = form == 0 ? 16 : (form == 1 ? 64 : 128);
     const int row_tiles = (P + rows - 1) / rows + E;
 #define MOE_GO(KERNEL, NB, TO) KERNEL<<<dim3((N + NB - 1) / NB, row_tiles), 256, 0, stream>>>((TO*)out, (const bf16_t*)a, (const bf16_t*)w, \
-        order, seg, E, top, gather, N, K, lda, act, scale)
+        order, seg, E, top, gather, N, K, lda, act, scale, row_weight)
     if (form == 0) { if (out_dtype == DT_F32) MOE_GO(moe_few_kernel<float>, 16, float); else MOE_GO(moe_few_kernel<bf16_t>, 16, bf16_t); }
     else if (form == 1) { if (out_dtype == DT_F32) MOE_GO((moe_tiles_kernel<64, 128, float>), 128, float); else MOE_GO((moe_tiles_kernel<64, 128, bf16_t>), 128, bf16_t); }
     else { if (out_dtype == DT_F32) MOE_GO((moe_tiles_kernel<128, 128, float>), 128, float); else MOE_GO((moe_tiles_kernel<128, 128, bf16_t>), 128, bf16_t); }

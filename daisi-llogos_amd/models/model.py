@@ -143,7 +143,12 @@ class Model:
         specs += self.final_norm.tensor_specs()
         if not s.tie_head:
             specs.append(TensorSpec(s.head_name + s.head_suffix, (s.vocab_size, s.hidden_size), "matrix"))
-        return specs
+        # a tensor that several parts read (a table whose columns the layers share out) is listed once
+        unique: Dict[str, TensorSpec] = {}
+        for spec in specs:
+            if unique.setdefault(spec.name, spec) != spec:
+                raise ValueError(f"two parts describe the tensor {spec.name} differently")
+        return list(unique.values())
 
     # ---- what the cache must hold ---------------------------------------------
     def cache_needs(self) -> List[Tuple[Optional[KVSpec], Optional[StateSpec]]]:

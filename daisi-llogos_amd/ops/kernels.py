@@ -637,12 +637,13 @@ def moe_route(ids: Optional[torch.Tensor], table: torch.Tensor, n_experts: int):
 
 
 def moe_router(h: torch.Tensor, router_w: torch.Tensor, correction: Optional[torch.Tensor], n_groups: int, keep: int, top: int,
-               scale: float):
+               scale: float, scores: str = "softmax", renorm: bool = True):
     """A router's choice for every row of h [T, K] (any storage type): logits z = h . router_w^T in 32-bit
     (router_w float32 [E, K]), s = softmax(z) over all E outputs, the choice's scores s + correction (float32 [E]
     or None), of which only those in the `keep` best of n_groups equal groups of neighbouring outputs (a group's
     score is its largest) can be chosen; the `top` largest are chosen (the lowest index among equals).
-    Returns (choice int32 [T, top], weight float32 [T, top]) with weight = s[choice] / (their sum + 1e-20) * scale."""
+    Returns (choice int32 [T, top], weight float32 [T, top]) with weight = s[choice] / (their sum + 1e-20) * scale.
+    scores "sigmoid": s is the logistic function of every logit by itself; renorm False: weight = s[choice] * scale."""
     _dev(router_w, correction)
     _need(h.is_cuda and h.dim() == 2 and h.stride(1) == 1, "moe_router: rows [T, K] on the GPU")
     _need(router_w.dtype == torch.float32 and router_w.dim() == 2 and router_w.shape[1] == h.shape[1], "moe_router: router_w must be float32 [E, K]")
@@ -650,6 +651,7 @@ def moe_router(h: torch.Tensor, router_w: torch.Tensor, correction: Optional[tor
     E = router_w.shape[0]
     _need(0 < top <= E <= MOE_MAX_EXPERTS, f"moe_router: top within 1..E, at most {MOE_MAX_EXPERTS} outputs")
     _need(correction is None or (correction.dtype == torch.float32 and correction.shape == (E,)), "moe_router: correction must be float32 [E]")
+    _need(scores in ("softmax", "sigmoid"), "moe_router: scores 'softmax' or 'sigmoid'")
     n_groups, keep = max(1, int(n_groups)), int(keep)
     if n_groups > 1:
         _need(E % n_groups == 0 and keep >= 1 and min(keep, n_groups) * (E // n_groups) >= top,
@@ -659,19 +661,23 @@ def moe_router(h: torch.Tensor, router_w: torch.Tensor, correction: Optional[tor
                                            T, E, Kk, _stream()), "moe_router_logits")
     choice = torch.empty((T, top), dtype=torch.int32, device=h.device)
     weight = torch.empty((T, top), dtype=torch.float32, device=h.device)
-    _check(_lib().llogos_moe_router_choose(_p(z), _p(correction), T, E, n_groups, keep, top, ctypes.c_float(scale), _p(choice),
-                                           _p(weight), _stream()), "moe_router_choose")
+    _check(_lib().llogos_moe_router_choose(_p(z), _p(correction), T, E, n_groups, keep, top, ctypes.c_float(scale),
+                                           int(scores == "sigmoid"), int(bool(renorm)), _p(choice), _p(weight), _stream()), "moe_router_choose")
     return choice, weight
 
 
-def moe_combine_weighted(y: torch.Tensor, where: torch.Tensor, choice: torch.Tensor, weight: torch.Tensor, n_real: int,
-                         h: torch.Tensor, shared: Optional[torch.Tensor] = None) -> torch.Tensor:
+def moe_combine_weighted(y: torch.Tensor, where: torch.Tensor, choice: torch.Tensor, weight: Optional[torch.Tensor], n_real: int,
+                         h: torch.Tensor, shared: Optional[torch.Tensor] = None, stream: Optional[torch.Tensor] = None,
+                         rows: bool = False):
     """float32 [T, W]: sum_j weight[t, j] * row_j + shared[t], where row_j is the pair's row y[where[t * top + j]]
     when choice[t, j] < n_real and the token's own row h[t] otherwise (a router output that has no matrices and
-    returns its input).  y float32 [T * top, W]; h [T, W] of any storage type; shared float32 [T, W] or parts."""
-    _dev(y, where, choice, weight)
+    returns its input).  y float32 [T * top, W]; h [T, W] of any storage type; shared float32 [T, W] or parts.
+    weight None: every row counts once.  stream: the result joins this float32 [T, W] in place, and what comes back is
+    None or, with `rows`, the new rows in h's type."""
+    _dev(y, where, choice, weight, stream)
     _i32(where, "where"); _i32(choice, "choice")
-    _need(choice.dim() == 2 and weight.shape == choice.shape and weight.dtype == torch.float32, "moe_combine_weighted: choice and weight [T, top]")
+    _need(choice.dim() == 2 and (weight is None or (weight.shape == choice.shape and weight.dtype == torch.float32)),
+          "moe_combine_weighted: choice and weight [T, top]")
     T, top = choice.shape
     _need(y.dtype == torch.float32 and y.dim() == 2 and y.shape[0] == T * top and where.numel() == T * top, "moe_combine_weighted: y float32 [T * top, W]")
     W = y.shape[1]
@@ -681,20 +687,26 @@ def moe_combine_weighted(y: torch.Tensor, where: torch.Tensor, choice: torch.Ten
         _dev(shared)
         parts, part_stride = _parts(shared)
         _need(shared.dtype == torch.float32 and tuple(shared.shape[-2:]) == (T, W), "moe_combine_weighted: shared rows float32 [T, W]")
-    out = torch.empty((T, W), dtype=torch.float32, device=y.device)
+    _need(stream is None or (stream.dtype == torch.float32 and stream.shape == (T, W)), "moe_combine_weighted: the stream must be float32 [T, W]")
+    _need(stream is not None or not rows, "moe_combine_weighted: rows are the stream's")
+    out = torch.empty((T, W), dtype=torch.float32, device=y.device) if stream is None else stream
+    new_rows = torch.empty((T, W), dtype=h.dtype, device=y.device) if rows else None
     _check(_lib().llogos_moe_combine_weighted(_p(out), _p(y), _p(where), _p(choice), _p(weight), top, int(n_real), _p(h), _dt(h),
                                               h.stride(0) if T > 1 else max(W, h.stride(0)), _p(shared), parts,
-                                              ctypes.c_longlong(part_stride), T, W, _stream()), "moe_combine_weighted")
-    return out
+                                              ctypes.c_longlong(part_stride), T, W, 0 if stream is None else 1, _p(new_rows), _stream()),
+           "moe_combine_weighted")
+    return out if stream is None else new_rows
 
 
 def moe_product(a: torch.Tensor, w: torch.Tensor, order: torch.Tensor, seg: torch.Tensor, top: int, gather: bool,
-                out_dtype: torch.dtype, relu2: bool = False, scale: float = 1.0, gated: bool = False) -> torch.Tensor:
+                out_dtype: torch.dtype, relu2: bool = False, scale: float = 1.0, gated: bool = False,
+                pair_weight: Optional[torch.Tensor] = None) -> torch.Tensor:
     """[P, N]: sorted row r, which belongs to the expert e whose segment holds it, is a_row(r) . w[e]^T, with
     a_row(r) = a[order[r] // top] (gather: a holds the step's token rows) or a[r] (a is sorted already);
     w [E, N, K]; relu2 squares max(., 0) in the epilogue, scale multiplies the result.  gated: the rows of
     w[e] are gate and up rows in turn (gate 0, up 0, gate 1, ...) and the result is [P, N / 2], column i
-    silu(gate_i sum) * (up_i sum).  `seg` may hold more segments than w has experts: rows in those belong
+    silu(gate_i sum) * (up_i sum); pair_weight float32 [P] (with gated): pair p's row counts as pair_weight[p] times
+    itself, which multiplies both sums.  `seg` may hold more segments than w has experts: rows in those belong
     to choices without a matrix and are left unwritten."""
     _dev(a, w, order, seg)
     _i32(order, "order"); _i32(seg, "seg")
@@ -706,6 +718,9 @@ def moe_product(a: torch.Tensor, w: torch.Tensor, order: torch.Tensor, seg: torc
     _need(gather or a.shape[0] == P, "moe_product: sorted rows must be as many as pairs")
     _need(not gather or a.shape[0] * top == P, "moe_product: token rows times choices must be the pairs")
     _need(not gated or N % 2 == 0, "moe_product: gate and up rows in turn make an even number of rows")
+    if pair_weight is not None:
+        _dev(pair_weight)
+        _need(gated and pair_weight.dtype == torch.float32 and pair_weight.numel() == P, "moe_product: pair_weight float32 [P], with the gated epilogue")
     act = 2 if gated else (1 if relu2 else 0)
     out = torch.empty((P, N // 2 if gated else N), dtype=out_dtype, device=a.device)
     if a.dtype == torch.bfloat16 and MOE_PRODUCT != "plain" and a.stride(1) == 1:
@@ -715,12 +730,12 @@ def moe_product(a: torch.Tensor, w: torch.Tensor, order: torch.Tensor, seg: torc
         if MOE_PRODUCT in ("few", "tiles64", "tiles128"):
             form = ("few", "tiles64", "tiles128").index(MOE_PRODUCT)
         code = _lib().llogos_moe_product_bf16(_p(out), _DT[out_dtype], _p(a), _p(w), _p(order), _p(seg), E, top, 1 if gather else 0,
-                                              P, N, Kk, a.stride(0), act, ctypes.c_float(scale), form, _stream())
+                                              P, N, Kk, a.stride(0), act, ctypes.c_float(scale), _p(pair_weight), form, _stream())
         if code != -2:
             _check(code, "moe_product")
             return out
     _check(_lib().llogos_moe_product(_p(out), _DT[out_dtype], _p(a), _dt(a), _p(w), _dt(w), _p(order), _p(seg), E, top,
-                                     1 if gather else 0, P, N, Kk, a.stride(0), act, ctypes.c_float(scale), _stream()),
+                                     1 if gather else 0, P, N, Kk, a.stride(0), act, ctypes.c_float(scale), _p(pair_weight), _stream()),
            "moe_product")
     return out
 
@@ -757,12 +772,13 @@ def moe_combine(y: torch.Tensor, where: torch.Tensor, top: int, shared: Optional
 # ----------------------------------------------------------------------------
 def latent_prepare(ctx, kv: torch.Tensor, qfull: torch.Tensor, q_out: torch.Tensor, norm_w: torch.Tensor, eps: float,
                    cs: Optional[torch.Tensor], k_pool: torch.Tensor, v_pool: Optional[torch.Tensor], table: torch.Tensor,
-                   n_heads: int, dim: int, rot: int, rot_dims: int, rank: int, c_out: Optional[torch.Tensor] = None) -> None:
+                   n_heads: int, dim: int, rot: int, rot_dims: int, rank: int, c_out: Optional[torch.Tensor] = None,
+                   pairing: int = 1) -> None:
     """From kv float32 [T, rank + rot] and qfull float32 [T, heads * (dim + rot)]: the normed latent and
     the rotated shared key part go to the token's key row in the cache ([rank | rot | zeros]); each
     head's rotated query part goes to q_out[t, h, rank:] ([T, heads, hd], hd the cache's row width).  With a
     value pool the latent is also stored as the token's value row, and with c_out ([T, rank] of the cache's type)
-    as plain rows."""
+    as plain rows.  pairing 0: rotated dimension i is paired with i + rot_dims / 2, 1: 2i with 2i + 1."""
     _dev(q_out, norm_w, cs, k_pool, v_pool, table, ctx.tok_seq, ctx.tok_pos)
     _i32(table, "table")
     T = ctx.n_tokens
@@ -787,18 +803,20 @@ def latent_prepare(ctx, kv: torch.Tensor, qfull: torch.Tensor, q_out: torch.Tens
     ld = lambda t_, least: t_.stride(0) if T > 1 else max(least, t_.stride(0))
     _check(_lib().llogos_latent_prepare(_p(kv), ld(kv, rank + rot), _p(qfull), ld(qfull, n_heads * (dim + rot)), _p(q_out), _dt(q_out), _p(norm_w),
                                         ctypes.c_float(eps), _p(cs), _p(k_pool), _p(v_pool), _p(table), table.stride(0), _p(ctx.tok_seq),
-                                        _p(ctx.tok_pos), T, n_heads, dim, rot, rot_dims, rank, hd, _p(c_out), _stream()), "latent_prepare")
+                                        _p(ctx.tok_pos), T, n_heads, dim, rot, rot_dims, int(pairing), rank, hd, _p(c_out), _stream()), "latent_prepare")
 
 
 LATENT_MFMA_MAX_ROW = 576
 
 
 def latent_attention_mfma(ctx, q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, table: torch.Tensor,
-                          n_heads: int, row: int, dv: int, scale: float, head_sink: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
+                          n_heads: int, row: int, dv: int, scale: float, head_sink: Optional[torch.Tensor],
+                          window: int = 0) -> Optional[torch.Tensor]:
     """bfloat16 attention over a latent cache on the matrix cores: q [T, heads, row], key rows and value rows
     (the latent in the value pages' order) in pools [pages, 1, 64 * row]; returns [T, heads, dv], or None
     for rows wider than the kernel takes.  Single-token steps share a sequence's pages out over several
-    blocks (chosen from the batch and the longest context the step may have) and merge."""
+    blocks (chosen from the batch and the longest context the step may have) and merge.  window > 0: a query
+    sees the last `window` keys, its own among them."""
     if q.dtype != torch.bfloat16 or row > LATENT_MFMA_MAX_ROW:
         return None
     T = ctx.n_tokens
@@ -816,6 +834,8 @@ def latent_attention_mfma(ctx, q: torch.Tensor, k_pool: torch.Tensor, v_pool: to
         _need(T == ctx.batch, "latent attention: a single-token step has one token a sequence")
         n_tiles = T * (-(-n_heads // 16))
         pages = max(1, min(table.shape[1], -(-ctx.max_context // PAGE_TOKENS)))
+        if window > 0:
+            pages = min(pages, -(-(window - 1) // PAGE_TOKENS) + 1)      # that a window can reach into
         want = max(1, (4 * compute_units()) // max(1, n_tiles))          # blocks of one wave's work: a few a compute unit
         pps = max(1, -(-pages // min(pages, want, 16)))                  # (the merge kernel takes up to 16 parts)
         splits = -(-pages // pps)
@@ -829,7 +849,7 @@ def latent_attention_mfma(ctx, q: torch.Tensor, k_pool: torch.Tensor, v_pool: to
         n_tiles = sum(-(-(ctx.cu_seqlens[i + 1] - ctx.cu_seqlens[i]) * n_heads // 16) for i in range(ctx.batch))
     out = torch.empty((T, n_heads, dv), dtype=torch.bfloat16, device=q.device)
     code = lib.llogos_latent_attn_bf16(_p(out), dv, _p(q), _p(k_pool), _p(v_pool), _p(table), table.stride(0), _p(cu),
-                                       _p(ctx.tok_pos), ctx.batch, T, n_heads, row, ctypes.c_float(scale), _p(head_sink),
+                                       _p(ctx.tok_pos), ctx.batch, T, n_heads, row, ctypes.c_float(scale), int(window), _p(head_sink),
                                        n_tiles, splits, pps, _p(ws), ctypes.c_longlong(ws.numel() if ws is not None else 0), _stream())
     if code == -2:
         return None
@@ -1055,6 +1075,119 @@ def diff_attention(ctx, q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Ten
         _p(out), _p(q), _dt(q), q.stride(0), _p(k_pool), _p(v_pool), _p(table), table.stride(0), _p(ctx.tok_seq), _p(ctx.tok_pos),
         T, n_heads, n_kv_heads, dim, v_dim, kd, vd, ctypes.c_float(scale), int(window), int(sinks), ctypes.c_float(lam),
         ctypes.c_float(out_scale), ctypes.c_float(eps), _stream()), "diff_attention_generic")
+    return out
+
+
+# ----------------------------------------------------------------------------
+# a recurrence with a fixed decay a head; sums into the stream; a table's row behind a gate
+# ----------------------------------------------------------------------------
+DECAY_CHUNK = 32             # tokens a chunk of the recurrence (kDecayChunk in csrc/decay_recurrence.hip)
+DECAY_SCAN_MAX_DIM = 256     # key channels a head
+DECAY_SEGMENTS = 0           # 0: chosen by the step; 1, 2, 3, ... force the number of segments of a prompt (tests)
+
+
+def decay_powers(decay: Sequence[float], device) -> torch.Tensor:
+    """float32 [heads, DECAY_CHUNK + 1]: the powers 0 .. DECAY_CHUNK of every head's decay, made in double."""
+    return torch.tensor([[float(a) ** n for n in range(DECAY_CHUNK + 1)] for a in decay], dtype=torch.float64).to(device=device, dtype=torch.float32).contiguous()
+
+
+def decay_segments(lens: Sequence[int], n_heads: int, col_blocks: int, n_cus: Optional[int] = None) -> Tuple[int, int]:
+    """(segments a sequence, tokens a segment) of the recurrence over a step's sequences: as many as bring the blocks
+    to about two a compute unit, of at least four chunks; segments cost the longer sequences a second pass over k and v."""
+    longest = max(lens)
+    n_cus = n_cus or compute_units()
+    want = DECAY_SEGMENTS or max(1, min(longest // (4 * DECAY_CHUNK), -(-2 * n_cus // max(1, len(lens) * n_heads * col_blocks))))
+    seg_len = -(-(-(-longest // want)) // DECAY_CHUNK) * DECAY_CHUNK
+    return -(-longest // seg_len), seg_len
+
+
+def decay_scan(ctx, rows: torch.Tensor, powers: torch.Tensor, state: torch.Tensor, n_heads: int, dim: int, v_dim: int) -> torch.Tensor:
+    """The recurrence S <- a S + k v^T, o = S^T q per head over the step's rows of each sequence in turn, with q, k, v the
+    silu of rows [q | k | v | ...] (float32 [T, >= W] or partial sums [parts, T, >= W], W = n_heads * (2 dim + v_dim));
+    powers: decay_powers of the heads' a; state float32 [slots, n_heads * dim * v_dim]: each head's S as
+    [key channel][value channel], read and brought up to date.  Returns o, float32 [T, n_heads * v_dim]."""
+    _dev(powers, state, ctx.slots, ctx.cu_dev)
+    _need(rows.is_cuda and rows.dtype == torch.float32 and rows.stride(-1) == 1, "decay_scan: float32 rows on the GPU")
+    parts, part_stride = _parts(rows)
+    T, W = rows.shape[-2], n_heads * (2 * dim + v_dim)
+    _need(T == ctx.n_tokens and rows.shape[-1] >= W, f"decay_scan: rows of at least {W} values, one a token")
+    _need(0 < dim <= DECAY_SCAN_MAX_DIM and v_dim > 0, f"decay_scan: at most {DECAY_SCAN_MAX_DIM} key channels a head")
+    _need(powers.dtype == torch.float32 and powers.shape == (n_heads, DECAY_CHUNK + 1), "decay_scan: the heads' powers")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.shape[1] == n_heads * dim * v_dim,
+          "decay_scan: state must be float32 [slots, heads * dim * v_dim]")
+    _need(ctx.cu_dev is not None or T == ctx.batch, "decay_scan: a step of several tokens a sequence needs the token offsets")
+    o = torch.empty((T, n_heads * v_dim), dtype=torch.float32, device=rows.device)
+    cu, n_seg, seg_len, seg_state, cols = None, 1, 0, None, 64
+    if ctx.is_decode or ctx.cu_dev is None:
+        # columns of the state a block: as few as bring the blocks to one a compute unit
+        cols = min(256, -(-v_dim // 4) * 4)
+        while cols > 16 and ctx.batch * n_heads * -(-v_dim // cols) < compute_units():
+            cols = -(-cols // 8) * 4
+    else:
+        cu = ctx.cu_dev
+        lens = [ctx.cu_seqlens[i + 1] - ctx.cu_seqlens[i] for i in range(ctx.batch)]
+        n_seg, seg_len = decay_segments(lens, n_heads, -(-v_dim // (128 if v_dim > 64 else 64)))
+        if n_seg > 1:
+            seg_state = torch.empty((ctx.batch, n_seg, n_heads, dim, v_dim), dtype=torch.float32, device=rows.device)
+    ld = rows.stride(-2) if T > 1 else max(W, rows.stride(-2))
+    _check(_lib().llogos_decay_scan(_p(o), _p(rows), ld, parts, ctypes.c_longlong(part_stride), _p(powers), _p(state),
+                                    ctypes.c_longlong(state.stride(0)), _p(ctx.slots), _p(cu), ctx.batch, n_heads, dim, v_dim, cols,
+                                    n_seg, seg_len, _p(seg_state), _stream()), "decay_scan")
+    return o
+
+
+def gated_row_norm(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
+    """o / sqrt(mean(o^2) + eps) * weight * sigmoid(gate) row by row: float32 o [T, N], weight [N]; gate float32 logits [T, N]
+    (maybe columns of wider rows) or partial sums [parts, T, N] of them."""
+    _dev(o, weight)
+    _need(o.dtype == torch.float32 and o.dim() == 2, "gated_row_norm: o must be float32 [T, N]")
+    T, N = o.shape
+    _need(weight.dtype == torch.float32 and weight.shape == (N,), "gated_row_norm: weight must be float32 [N]")
+    parts, part_stride = _parts(gate)
+    _need(gate.is_cuda and gate.dtype == torch.float32 and tuple(gate.shape[-2:]) == (T, N) and gate.stride(-1) == 1,
+          "gated_row_norm: gate must be float32 [T, N]")
+    y = torch.empty((T, N), dtype=out_dtype, device=o.device)
+    if T:
+        _check(_lib().llogos_gated_row_norm(_p(y), _DT[out_dtype], _p(o), _p(weight), _p(gate), gate.stride(-2) if T > 1 else max(N, gate.stride(-2)),
+                                            parts, ctypes.c_longlong(part_stride), ctypes.c_float(eps), T, N, _stream()), "gated_row_norm")
+    return y
+
+
+def stream_add(x: torch.Tensor, delta: Optional[torch.Tensor] = None, again: Optional[torch.Tensor] = None,
+               vector: Optional[torch.Tensor] = None, rows_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
+    """In place on the float32 stream x [T, W]: x += delta ([T, W] or partial sums [parts, T, W]) + again (float32 [T, W]) +
+    vector (float32 [W], the same for every row), each of which may be absent.  With rows_dtype the new rows come back in
+    that type (for float32 that is x itself)."""
+    _dev(x, delta, again, vector)
+    _need(x.dtype == torch.float32 and x.dim() == 2, "stream_add: the stream must be float32 [T, W]")
+    T, W = x.shape
+    parts, part_stride = _parts(delta)
+    if delta is not None:
+        _need(tuple(delta.shape[-2:]) == (T, W) and (parts == 1 or delta.dtype == torch.float32), "stream_add: delta must be [T, W] or float32 parts of it")
+    _need(again is None or (again.dtype == torch.float32 and again.shape == (T, W)), "stream_add: again must be float32 [T, W]")
+    _need(vector is None or (vector.dtype == torch.float32 and vector.shape == (W,)), "stream_add: vector must be float32 [W]")
+    rows = None
+    if rows_dtype is not None and rows_dtype != torch.float32:
+        rows = torch.empty((T, W), dtype=rows_dtype, device=x.device)
+    if T and not (delta is None and again is None and vector is None and rows is None):
+        _check(_lib().llogos_stream_add(_p(x), _p(delta), _dt(delta) if delta is not None else F32, parts, ctypes.c_longlong(part_stride),
+                                        _p(again), _p(vector), _p(rows), _dt(rows) if rows is not None else F32, T, W, _stream()), "stream_add")
+    return x if rows_dtype == torch.float32 else rows
+
+
+def gated_lookup(z: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """gelu_tanh(z[t]) * table[ids[t]]: z [T, N] or float32 partial sums [parts, T, N], table [V, N] in the output's type,
+    int32 ids [T]."""
+    _dev(z, table, ids)
+    _i32(ids, "ids")
+    parts, part_stride = _parts(z)
+    T, N = z.shape[-2:]
+    _need(table.dim() == 2 and table.shape[1] == N and table.dtype == out_dtype, "gated_lookup: table [V, N] in the output's type")
+    _need(ids.numel() == T and (z.dtype == torch.float32 or (parts == 1 and z.dtype == out_dtype)), "gated_lookup: one id a row; z float32 or the output's type")
+    out = torch.empty((T, N), dtype=out_dtype, device=z.device)
+    if out.numel():
+        _check(_lib().llogos_gated_lookup(_p(out), _DT[out_dtype], _p(z), _dt(z), parts, ctypes.c_longlong(part_stride), _p(table), _dt(table),
+                                          _p(ids), T, N, _stream()), "gated_lookup")
     return out
 
 

@@ -12,7 +12,9 @@ from .latent_attention import LatentAttention
 from .mlp import ActivatedMLP, SwiGLU
 from .capped_attention import CappedAttention
 from .moe import RoutedMoE, TableMoE
-from .loop import LoopEntry
+from .loop import LoopAdd, LoopEntry
+from .token_side import TokenSide
+from .lightning import Lightning
 from .rglru import RGLRU
 from .diff_attention import DiffAttention
 from .block import OutputNormBlock, ParallelBlock, PostNormBlock, PreNormBlock, SandwichBlock

@@ -253,6 +253,14 @@ class Norm(Part):
     # norm that reads it next says so.
     takes_row_squares = False
 
+    # True for a reader of the stream that is no norm but takes the stream's own rows (row_weight() is all ones):
+    # whoever completes the stream may leave them as RowSquares.unscaled without the sums of squares
+    plain_rows = False
+
+    # True when the reader of this norm's rows takes them as float32 (set by the block that holds both, for
+    # whoever prepares the rows in advance)
+    float32_rows = False
+
     def row_weight(self) -> Optional[torch.Tensor]:
         """float32 [H]: the weight w of a norm of the form x * w * (a scale of the whole row from the
         row's mean square and eps); None for any other norm."""

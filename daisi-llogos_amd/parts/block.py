@@ -15,22 +15,30 @@ from typing import Callable, List, Optional, Tuple
 import torch
 
 from .base import Block, FeedForward, LayerCache, Mixer, Norm, NormedAhead, Part, Residual, Runtime, StepContext, TensorSpec, mark, register_block
-from .norm import RMSNorm
+from .norm import RMSNorm, add_normed
 
 
 @register_block("pre_norm")
 class PreNormBlock(Block):
-    def __init__(self, mixer_norm: Norm, mixer: Mixer, ffn_norm: Norm, ffn: FeedForward):
-        self.mixer_norm, self.mixer, self.ffn_norm, self.ffn = mixer_norm, mixer, ffn_norm, ffn
+    """The feed-forward may be absent (its norm's tensor may be there all the same; nothing reads it).  `tail`: a
+    part that transforms the stream behind the feed-forward, forward(ctx, x, pending, next_norm) -> (x, pending)."""
+
+    def __init__(self, mixer_norm: Norm, mixer: Mixer, ffn_norm: Optional[Norm] = None, ffn: Optional[FeedForward] = None,
+                 tail: Optional[Part] = None):
+        if ffn is not None and ffn_norm is None:
+            raise ValueError("a feed-forward comes with the norm in front of it")
+        self.mixer_norm, self.mixer, self.ffn_norm, self.ffn, self.tail = mixer_norm, mixer, ffn_norm, ffn, tail
+        if mixer.takes_float32_rows:
+            mixer_norm.float32_rows = True
 
     def mixers(self) -> List[Mixer]:
         return [self.mixer]
 
     def feed_forwards(self) -> List[FeedForward]:
-        return [self.ffn]
+        return [self.ffn] if self.ffn is not None else []
 
     def parts(self) -> List[Part]:
-        return [self.mixer_norm, self.mixer, self.ffn_norm, self.ffn]
+        return [p for p in (self.mixer_norm, self.mixer, self.ffn_norm, self.ffn, self.tail) if p is not None]
 
     takes_next_norm = True
 
@@ -39,6 +47,8 @@ class PreNormBlock(Block):
 
     @staticmethod
     def _norm(norm: Norm, x: torch.Tensor, delta, lazy: bool):
+        if norm.float32_rows:
+            return norm.forward(x, delta, out_dtype=torch.float32)
         # (only a norm that knows of unscaled rows is asked for them)
         return norm.forward(x, delta, lazy=True) if lazy and norm.takes_row_squares else norm.forward(x, delta)
 
@@ -46,21 +56,20 @@ class PreNormBlock(Block):
         cache = caches[0] if isinstance(caches, (list, tuple)) else caches
         # A part that says so may add its output to x itself and leave the next norm's rows half made
         # (then `a` or `d` is what it left, and the norm that takes it needs no kernel of its own).
+        last = self.tail if self.tail is not None else next_norm            # who reads the stream behind the sublayers
+
+        def closing(part, reader):
+            return dict(residual=Residual(x, reader)) if part.adds_to_residual and reader is not None and reader.takes_row_squares else {}
         h = self._norm(self.mixer_norm, x, pending, self.mixer.takes_normed_rows)
         mark(ctx, "norm")
-        if self.mixer.adds_to_residual and self.ffn_norm.takes_row_squares:
-            a = self.mixer.forward(ctx, h, cache, residual=Residual(x, self.ffn_norm))
-        else:
-            a = self.mixer.forward(ctx, h, cache)
+        d = self.mixer.forward(ctx, h, cache, **closing(self.mixer, self.ffn_norm if self.ffn is not None else last))
         mark(ctx, "mixer")
-        h = self._norm(self.ffn_norm, x, a, self.ffn.takes_normed_rows)
-        mark(ctx, "norm")
-        if self.ffn.adds_to_residual and next_norm is not None and next_norm.takes_row_squares:
-            d = self.ffn.forward(ctx, h, residual=Residual(x, next_norm))
-        else:
-            d = self.ffn.forward(ctx, h)
-        mark(ctx, "feed_forward")
-        return x, d
+        if self.ffn is not None:
+            h = self._norm(self.ffn_norm, x, d, self.ffn.takes_normed_rows)
+            mark(ctx, "norm")
+            d = self.ffn.forward(ctx, h, **closing(self.ffn, last))
+            mark(ctx, "feed_forward")
+        return (x, d) if self.tail is None else self.tail.forward(ctx, x, d, next_norm)
 
 
 @register_block("sandwich")
@@ -115,19 +124,10 @@ class SandwichBlock(Block):
 
     def _close(self, x, out, post: Norm, nxt: Optional[Norm], rows_f32: bool):
         """A sublayer's output `out` joins the stream through its norm `post`, and the norm `nxt` that
-        reads the stream next is applied on the way: one kernel for both where both are RMS norms over the
-        stream's width (then x is complete and the rows are returned), else the norm's own kernel (then the
-        normed output is returned as a delta that the next norm adds).  Returns (rows or None, delta or None).
+        reads the stream next is applied on the way (add_normed).  Returns (rows or None, delta or None).
         The rows handed to another block are float32 (a convolution or a mixer that mixes rows reads them)."""
-        from ..ops import kernels as K
-        fused = isinstance(post, RMSNorm) and (nxt is None or isinstance(nxt, RMSNorm)) and x.shape[1] * 4 <= 65536 \
-            and (nxt is None or nxt.eps == post.eps)
-        if not fused:
-            a = out if (out.dim() == 2 and out.dtype == torch.float32) else K.sum_parts(out, None, torch.float32)
-            return None, post.forward(a, out_dtype=torch.float32)
-        dtype = torch.float32 if rows_f32 else self.rt.dtype
-        rows = K.sandwich_norm(x, out, post.weight, nxt.weight if nxt is not None else None, post.eps, dtype)
-        return rows, None
+        made = add_normed(x, out, post, nxt, torch.float32 if rows_f32 else self.rt.dtype)
+        return (made.rows, None) if isinstance(made, NormedAhead) else (None, made)
 
     def forward(self, ctx: StepContext, x: torch.Tensor, pending, caches, next_norm: Optional[Norm] = None):
         caches = list(caches)

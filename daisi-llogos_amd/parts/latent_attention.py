@@ -1,11 +1,11 @@
-"""Attention through a low-rank latent, with an optional learned sink in the softmax and an optional
-sigmoid gate on every head's output.
+"""Attention through a low-rank latent, with an optional learned sink in the softmax, an optional
+sigmoid gate on every head's output and an optional sliding window.
 
     c_q = norm(W_dq h);  q = W_uq c_q                    per head [dim unrotated | rot rotated]
                                                          (q_rank 0: q = W_q h, no latent on the query's side)
     [c_raw | k_rot] = W_dkv h;  c = norm(c_raw)          the latent, and one rotated key part for all heads
     k_h = W_uk,h c;  v_h = W_uv,h c
-    score_h(i, j) = (q_h,plain(i) . k_h(j) + q_h,rot(i) . k_rot(j)) * scale,   j <= i
+    score_h(i, j) = (q_h,plain(i) . k_h(j) + q_h,rot(i) . k_rot(j)) * scale,   j <= i [and i - j < window]
     weights = exp(score) / (sum_j exp(score) [+ exp(sink_h)])
     out = W_o [sigmoid(W_g h)_h * sum_j weights_h(i, j) v_h(j)]_h            (the gate is optional)
 
@@ -27,7 +27,7 @@ from typing import Callable, List, Optional
 import torch
 
 from ..ops import kernels as K
-from .base import KVSpec, LayerCache, Mixer, Runtime, StepContext, TensorSpec, mark, register_mixer
+from .base import KVSpec, LayerCache, Mixer, Residual, Runtime, StepContext, TensorSpec, mark, register_mixer
 from .linear import Linear
 from .rope import Rotary
 
@@ -35,18 +35,23 @@ from .rope import Rotary
 @register_mixer("latent_attention")
 class LatentAttention(Mixer):
     graph_safe = True
+    adds_to_residual = True
 
     def __init__(self, prefix: str, hidden: int, n_heads: int, dim: int, rot_dim: int, v_dim: int, q_rank: int,
                  kv_rank: int, scale: float, eps: float, position: Optional[Rotary] = None, sink: bool = True,
-                 suffix: str = "", head_gate: bool = False):
+                 suffix: str = "", head_gate: bool = False, window: int = 0):
+        """window > 0: a query sees the last `window` positions, its own among them."""
         self.prefix, self.hidden = prefix, int(hidden)
         self.n_heads, self.dim, self.rot_dim, self.v_dim = int(n_heads), int(dim), int(rot_dim), int(v_dim)
         self.q_rank, self.kv_rank = int(q_rank), int(kv_rank)
         self.scale, self.eps = float(scale), float(eps)
         self.position = position
         self.has_sink, self.head_gate = bool(sink), bool(head_gate)
-        if position is not None and (position.pairing != 1 or position.rot > self.rot_dim):
-            raise ValueError("the rotated key part takes neighbouring pairs, at most rot_dim dimensions")
+        self.window = int(window)
+        if position is not None and position.rot > self.rot_dim:
+            raise ValueError("the rotated key part has rot_dim dimensions")
+        if self.window < 0:
+            raise ValueError(f"a window of {window}")
         # the cached row [latent | rotated part], widened to the pages' step of 16 dimensions
         self.row = -(-(self.kv_rank + self.rot_dim) // K.HEAD_DIM_STEP) * K.HEAD_DIM_STEP
         if self.row > 1024:
@@ -80,7 +85,7 @@ class LatentAttention(Mixer):
         # own: the latent is then cached a second time, as a value row; otherwise a value is part of its key row
         rt = getattr(self, "rt", None)
         mfma = rt is not None and rt.dtype == torch.bfloat16 and self.row <= K.LATENT_MFMA_MAX_ROW
-        return KVSpec(1, self.row, values=mfma)
+        return KVSpec(1, self.row, window=self.window, values=mfma)
 
     def tensor_specs(self) -> List[TensorSpec]:
         p, H = self.prefix, self.n_heads
@@ -119,7 +124,7 @@ class LatentAttention(Mixer):
 
     def _heads_on_matrix_cores(self) -> bool:
         """Whether whole prompts can run as attention with keys and values a head (see the module's text)."""
-        return self.rt.dtype == torch.bfloat16 and self.rot_dim == 0 and not self.q_rank and self.dim in (64, 96, 128) \
+        return self.rt.dtype == torch.bfloat16 and self.rot_dim == 0 and self.window == 0 and not self.q_rank and self.dim in (64, 96, 128) \
             and self.v_dim in (64, 80, 96, 128)
 
     @staticmethod
@@ -136,7 +141,15 @@ class LatentAttention(Mixer):
             made = ctx.shared["prompt_pages"] = (sum(pages), table)
         return made
 
-    def _forward_prompt(self, ctx: StepContext, rows: torch.Tensor, kv: torch.Tensor, gate, cache: LayerCache) -> torch.Tensor:
+    def _close(self, ctx: StepContext, a: torch.Tensor, residual: Optional[Residual]):
+        out = self.o.add_to(a, residual) if residual is not None else None
+        if out is None:
+            out = self.o.product(a, f32_ok=True)
+        mark(ctx, "o")
+        return out
+
+    def _forward_prompt(self, ctx: StepContext, rows: torch.Tensor, kv: torch.Tensor, gate, cache: LayerCache,
+                        residual: Optional[Residual]):
         f32, H, T = torch.float32, self.n_heads, ctx.n_tokens
         qa = torch.empty((T, H, self.row), dtype=self.rt.dtype, device=rows.device)       # (no rotated part: nothing is written)
         c = torch.empty((T, self.kv_rank), dtype=self.rt.dtype, device=rows.device)
@@ -151,11 +164,9 @@ class LatentAttention(Mixer):
                           table, kv_rows=keys_values)
         a = K.capped_attention(ctx, q, k_pool, v_pool, table, H, H, self.dim, self.v_dim, self.scale, 0.0, self.sink, gate)
         mark(ctx, "attention")
-        out = self.o.product(a, f32_ok=True)
-        mark(ctx, "o")
-        return out
+        return self._close(ctx, a, residual)
 
-    def forward(self, ctx: StepContext, h: torch.Tensor, cache: LayerCache) -> torch.Tensor:
+    def forward(self, ctx: StepContext, h: torch.Tensor, cache: LayerCache, residual: Optional[Residual] = None):
         f32, H, T = torch.float32, self.n_heads, ctx.n_tokens
         plain = lambda p: K.sum_parts(p, None, f32)          # (a product may come as partial sums of a split along k)
         rows = plain(self.inp.product(h, f32_ok=True))                            # [T, (q) | rank + rot | (heads)]
@@ -170,22 +181,22 @@ class LatentAttention(Mixer):
         mark(ctx, "projections")
         if self.ukv is not None and not ctx.is_decode and not ctx.in_graph and T >= self.prompt_rows and ctx.cu_dev is not None \
                 and not any(ctx.starts):
-            return self._forward_prompt(ctx, rows, kv, gate, cache)
+            return self._forward_prompt(ctx, rows, kv, gate, cache, residual)
         cs = self.position.prepare(ctx) if self.position is not None else None
         qa = torch.empty((T, H, self.row), dtype=self.rt.dtype, device=h.device)
         K.latent_prepare(ctx, kv, q, qa, self.c_norm_w, self.eps, cs, cache.k_pool, cache.v_pool, cache.table, H, self.dim, self.rot_dim,
-                         self.position.rot if self.position is not None else 0, self.kv_rank)
+                         self.position.rot if self.position is not None else 0, self.kv_rank,
+                         pairing=self.position.pairing if self.position is not None else 1)
         K.head_products(q.unflatten(1, (H, self.dim + self.rot_dim))[:, :, :self.dim], self.uk_t, qa[:, :, :self.kv_rank], self.uk_kn)
         mark(ctx, "rotation")
         lat = None
         if cache.v_pool is not None:
-            lat = K.latent_attention_mfma(ctx, qa, cache.k_pool, cache.v_pool, cache.table, H, self.row, self.kv_rank, self.scale, self.sink)
+            lat = K.latent_attention_mfma(ctx, qa, cache.k_pool, cache.v_pool, cache.table, H, self.row, self.kv_rank, self.scale, self.sink,
+                                          self.window)
         if lat is None:
             lat = K.attention_generic(qa, H * self.row, cache.k_pool, None, cache.table, ctx.tok_seq, ctx.tok_pos, H, 1, self.row,
-                                      self.scale, v_dim=self.kv_rank, head_sink=self.sink)
+                                      self.scale, window=self.window, v_dim=self.kv_rank, head_sink=self.sink)
         mark(ctx, "attention")
         a = torch.empty((T, H, self.v_dim), dtype=self.rt.dtype, device=h.device)
         K.head_products(lat.view(T, H, self.kv_rank), self.uv, a, self.uv_kn, gate=gate)
-        out = self.o.product(a.view(T, H * self.v_dim), f32_ok=True)
-        mark(ctx, "o")
-        return out
+        return self._close(ctx, a.view(T, H * self.v_dim), residual)

@@ -4,7 +4,7 @@ vector is added,
 
     x <- W_in [x ; x0] + step[t]           W_in [width, 2 width] (x first), step [times, width], t the pass
 
-in front of the first layer of every pass, the first pass too."""
+in front of the first layer of every pass, the first pass too.  `LoopAdd` is the form without a matrix."""
 from __future__ import annotations
 
 from typing import Callable, List, Optional
@@ -40,3 +40,27 @@ class LoopEntry(Part):
         both = K.concat_rows(x, x0, self.rt.dtype, delta=pending, write_back=False)
         out = K.sum_parts(self.mix.product(both, f32_ok=True), self.steps[number], torch.float32)
         return out, None
+
+
+@register_part("loop_add")
+class LoopAdd(Part):
+    """The same place filled by sums alone: x <- x + step[t], from the second pass on also + x0."""
+
+    def __init__(self, steps: str, width: int, times: int):
+        self.width, self.times, self.steps_name = int(width), int(times), steps
+        self.steps: Optional[torch.Tensor] = None
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        return [TensorSpec(self.steps_name, (self.times, self.width), "bias")]
+
+    def bind(self, get: Callable[[str], Optional[torch.Tensor]], rt: Runtime) -> None:
+        super().bind(get, rt)
+        self.steps = get(self.steps_name).to(device=rt.device, dtype=torch.float32).contiguous()
+
+    def forward(self, ctx: StepContext, x: torch.Tensor, pending, x0: torch.Tensor, number: int):
+        if not 0 <= number < self.times:
+            raise ValueError(f"pass {number} of {self.times}")
+        if isinstance(pending, (NormedAhead, K.RowSquares)):
+            pending = None                         # the stream is complete already
+        K.stream_add(x, pending, again=x0 if number > 0 else None, vector=self.steps[number])
+        return x, None

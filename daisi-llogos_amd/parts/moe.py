@@ -15,7 +15,7 @@ from typing import Callable, List, Optional
 import torch
 
 from ..ops import kernels as K
-from .base import FeedForward, Runtime, StepContext, TensorSpec, mark, register_feed_forward
+from .base import FeedForward, Residual, Runtime, StepContext, TensorSpec, mark, register_feed_forward
 from .linear import Linear
 
 _EPILOGUES = ("relu2",)        # activations that the experts' product applies in its epilogue
@@ -107,6 +107,10 @@ class RoutedMoE(FeedForward):
         weights w_j = s_j / (sum of the chosen s + 1e-20) * scale
         out = sum_j w_j expert_j(h)  +  shared(h),     expert(h) = W_down (silu(W_gate h) * (W_up h))
 
+    Three options change the router: `scores="sigmoid"` takes the logistic function of every logit by itself, `renorm=False`
+    leaves the weights as the chosen scores (times scale), `weigh="input"` puts a choice's weight on its expert's input,
+    expert_j(w_j h), instead of its output.
+
     The last `identity` router outputs have no matrices: such an expert returns h itself.  The choice, the
     sorting of the (token, choice) pairs by expert and the weighted sum are made on the device, so single-token
     steps are captured and replayed.  An expert's gate and up matrices are stacked with their rows in turn
@@ -121,17 +125,24 @@ class RoutedMoE(FeedForward):
     2,429 -> 2,335 us and 1,529 -> 1,470 us a step; 2,048 wide with 50 MB 1,457 -> 1,469 and 1,012 -> 1,037), so it is
     taken from `side_bytes` of shared matrices on.  `LLOGOS_PARALLEL_STREAMS=0` keeps everything on one stream."""
     graph_safe = True
+    adds_to_residual = True
     side_rows = 0 if os.environ.get("LLOGOS_PARALLEL_STREAMS", "1") == "0" else 64     # steps of up to so many rows use the second stream
     side_bytes = 64 << 20        # ... when the shared expert's matrices take at least so many bytes
     _side_streams = {}
 
     def __init__(self, prefix: str, hidden: int, n_experts: int, top: int, intermediate: int, identity: int = 0,
-                 groups: int = 1, keep: int = 1, scale: float = 1.0, shared_intermediate: int = 0, correction: bool = True):
+                 groups: int = 1, keep: int = 1, scale: float = 1.0, shared_intermediate: int = 0, correction: bool = True,
+                 scores: str = "softmax", renorm: bool = True, weigh: str = "output"):
         total = int(n_experts) + int(identity)
         if not 1 <= top <= total <= K.MOE_MAX_EXPERTS:
             raise ValueError(f"top {top} of {total} router outputs: outside 1..outputs..{K.MOE_MAX_EXPERTS}")
+        if weigh == "input" and identity:
+            raise ValueError("router outputs without matrices take their weight on the output")
         if groups < 1 or total % groups or not 1 <= keep <= groups or keep * (total // groups) < top:
             raise ValueError(f"{groups} groups of which {keep} are kept do not fit {total} router outputs and top {top}")
+        if scores not in ("softmax", "sigmoid") or weigh not in ("output", "input"):
+            raise ValueError(f"scores '{scores}' (softmax, sigmoid), weigh '{weigh}' (output, input)")
+        self.scores, self.renorm, self.weigh = scores, bool(renorm), weigh
         self.prefix, self.hidden = prefix, int(hidden)
         self.n_experts, self.identity, self.top, self.intermediate = int(n_experts), int(identity), int(top), int(intermediate)
         self.groups, self.keep, self.scale = int(groups), int(keep), float(scale)
@@ -180,7 +191,7 @@ class RoutedMoE(FeedForward):
         """What a token is multiplied with: the router, its `top` experts (as if all had matrices) and the shared one."""
         return super().matrix_elements() + self.outputs * self.hidden + 3 * self.top * self.intermediate * self.hidden
 
-    def forward(self, ctx: StepContext, h: torch.Tensor):
+    def forward(self, ctx: StepContext, h: torch.Tensor, residual: Optional[Residual] = None):
         shared, side = None, None
         if self.shared is not None and h.shape[0] <= self.side_rows and (ctx is None or ctx.probe is None) and h.is_cuda \
                 and 3 * self.shared_intermediate * self.hidden * h.element_size() >= self.side_bytes:
@@ -191,14 +202,16 @@ class RoutedMoE(FeedForward):
             side.wait_stream(main)                       # h is there
             with torch.cuda.stream(side):
                 shared = _float32(self.shared.forward(ctx, h))
-        choice, weight = K.moe_router(h, self.router_w, self.correction, self.groups, self.keep, self.top, self.scale)
+        choice, weight = K.moe_router(h, self.router_w, self.correction, self.groups, self.keep, self.top, self.scale,
+                                      scores=self.scores, renorm=self.renorm)
         mark(ctx, "router")
         if ctx is not None and ctx.probe is not None:
             self.probed = {"choice": choice}
         T, W = h.shape
         if self.n_experts:
             order, seg, where = K.moe_route(None, choice, self.outputs)
-            act = K.moe_product(h, self.gate_up, order, seg, self.top, True, self.rt.dtype, gated=True)
+            act = K.moe_product(h, self.gate_up, order, seg, self.top, True, self.rt.dtype, gated=True,
+                                pair_weight=weight.view(-1) if self.weigh == "input" else None)
             y = K.moe_product(act, self.down, order, seg, self.top, False, torch.float32)
         else:
             where = torch.zeros(T * self.top, dtype=torch.int32, device=h.device)
@@ -209,6 +222,10 @@ class RoutedMoE(FeedForward):
         elif self.shared is not None:
             shared = _float32(self.shared.forward(ctx, h))
             mark(ctx, "shared")
-        out = K.moe_combine_weighted(y, where, choice, weight, self.n_experts, h, shared)
+        x = residual.x if residual is not None else None
+        rows = x is not None and residual.norm is not None and residual.norm.plain_rows
+        out = K.moe_combine_weighted(y, where, choice, weight if self.weigh == "output" else None, self.n_experts, h, shared,
+                                     stream=x, rows=rows and not self.rt.is_f32)
         mark(ctx, "combine")
-        return out
+        # (added to the stream: what is left is its rows, for a reader that takes them as they are)
+        return out if x is None else K.RowSquares(None, W, out, residual.norm.row_weight() if rows else None)

@@ -12,6 +12,21 @@ from ..ops import kernels as K
 from .base import Norm, NormedAhead, NormedRows, Runtime, TensorSpec, register_norm
 
 
+def add_normed(x: torch.Tensor, out: torch.Tensor, post: Norm, nxt: Optional[Norm], dtype: Optional[torch.dtype] = None):
+    """The stream x (float32, in place) += post(out), and the rows that the norm `nxt` makes of the completed
+    stream on the way: one kernel where both are RMS norms over the stream's width; then a NormedAhead comes
+    back, with rows in `dtype` (None: the type that nxt's reader takes; without nxt there are none).  Otherwise
+    post's own kernel: its rows come back as a float32 delta that the stream still lacks."""
+    fused = isinstance(post, RMSNorm) and (nxt is None or (isinstance(nxt, RMSNorm) and nxt.eps == post.eps)) and x.shape[1] * 4 <= 65536
+    if not fused:
+        a = out if (out.dim() == 2 and out.dtype == torch.float32) else K.sum_parts(out, None, torch.float32)
+        return post.forward(a, out_dtype=torch.float32)
+    if dtype is None:
+        dtype = torch.float32 if nxt is None or nxt.float32_rows else post.rt.dtype
+    rows = K.sandwich_norm(x, out, post.weight, nxt.weight if nxt is not None else None, post.eps, dtype)
+    return NormedAhead(rows, nxt)
+
+
 @register_norm("rmsnorm")
 class RMSNorm(Norm):
     takes_row_squares = True

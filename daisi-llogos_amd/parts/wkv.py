@@ -19,7 +19,7 @@ from typing import Callable, List, Optional
 import torch
 
 from ..ops import kernels as K
-from .base import LayerCache, Mixer, Runtime, StateSpec, StepContext, TensorSpec, mark, register_mixer
+from .base import LayerCache, Mixer, Residual, Runtime, StateSpec, StepContext, TensorSpec, mark, register_mixer
 from .linear import Linear
 
 MIXES = ("r", "k", "v", "g", "w")
@@ -28,6 +28,7 @@ MIXES = ("r", "k", "v", "g", "w")
 @register_mixer("wkv")
 class WKV(Mixer):
     graph_safe = True
+    adds_to_residual = True
     takes_float32_rows = True        # the mixes are made from the unrounded rows
 
     def __init__(self, prefix: str, hidden: int, n_heads: int, head_dim: int, decay_rank: int, eps: float, suffix: str = ""):
@@ -65,7 +66,7 @@ class WKV(Mixer):
         self.mu = torch.stack([f32("mu." + s) for s in MIXES]).contiguous()
         self.w0, self.u, self.norm_w = f32("w0"), f32("u").reshape(-1), f32("norm")
 
-    def forward(self, ctx: StepContext, h: torch.Tensor, cache: LayerCache) -> torch.Tensor:
+    def forward(self, ctx: StepContext, h: torch.Tensor, cache: LayerCache, residual: Optional[Residual] = None):
         f32 = torch.float32
         state = cache.state
         prev = state[:, self.inner * self.head_dim:]
@@ -81,6 +82,8 @@ class WKV(Mixer):
         y = K.wkv_scan(ctx, r, k, v, d, g, self.w0, self.u, self.norm_w, self.eps, state, self.n_heads, self.head_dim,
                        h, self.rt.dtype)
         mark(ctx, "recurrence")
-        out = self.o.product(y, f32_ok=True)          # maybe in parts: the norm that follows adds them
+        out = self.o.add_to(y, residual) if residual is not None else None
+        if out is None:
+            out = self.o.product(y, f32_ok=True)      # maybe in parts: the norm that follows adds them
         mark(ctx, "o")
         return out
