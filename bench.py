@@ -219,6 +219,27 @@ def zasidra_config(width, layers, vocab, ff):
             "layers": out, "torch_dtype": "bfloat16"}
 
 
+def peponex_config(width, runs, vocab, ff):
+    """Layers of real sizes: a token-made decay recurrence in front and behind, between them fixed-decay recurrences and
+    latent attention in turn, the first such pair gone through twice, which makes `runs` runs of `runs - 2` layers.  Heads
+    of 64 channels in the first recurrence and of 128 in the second; attention with 128 + 64 query/key dimensions a
+    head, values of 128, a latent of 512 and a window of 1,024; feed-forwards dense and a mixture in turn, 16 experts of
+    which a token takes 2, each half as wide as the dense feed-forward; a token's part of 256 values a layer."""
+    heads = width // 128
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "router": {"experts": 16, "top": 2}, "expert": {"ff": ff // 2}}
+    wkv = {"type": "wkv", "mixer": {"heads": width // 64, "dim": 64, "decay_rank": 64}}
+    lig = {"type": "lightning", "mixer": {"heads": heads, "dim": 128, "vdim": 128,
+                                          "decay": [1.0 - 2.0 ** (-1.0 - 8.0 * (h + 1) / heads) for h in range(heads)]}}
+    lat = {"type": "latent_attention",
+           "mixer": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
+                     "mask": {"size": 1024}, "rot": {"base": 10000.0, "dims": 64}}}
+    n = runs - 2
+    layers = [dict(wkv, mlp=dense)] + [dict(lig, mlp=moe) if i % 2 == 0 else dict(lat, mlp=dense) for i in range(n - 2)] + [dict(wkv, mlp=moe)]
+    return {"architecture": "Peponex", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "logit_softcap": 30.0,
+            "token_side": {"dim": 256}, "loop": {"start": 1, "stop": 3, "times": 2}, "layers": layers, "torch_dtype": "bfloat16"}
+
+
 def moe_bytes_read(model, ids) -> int:
     """Bytes of weights that a step with the token ids `ids` reads: as step_weight_bytes, but of a layer's experts
     only those that the layer's table names for these ids, or that its router chose in the last step that was
@@ -285,7 +306,7 @@ def compare_designs(args) -> int:
             eng.step([(x, toks(args.prompt_len)) for x in slots], want="last")
             ids = toks(batch)                                     # a token of its own for every sequence (an expert choice of its own)
             step = lambda: eng.step([(x, [t]) for x, t in zip(slots, ids)], want="last", borrow=True)
-            if args.design == "zasidra" and label.startswith("zasidra"):
+            if label.split()[0] in ("zasidra", "peponex"):
                 # a step run part by part leaves every router's choice behind: the experts that such a step reads
                 eng.step([(x, [t]) for x, t in zip(slots, ids)], want="last", probe=llogos.StepProbe())
             for _ in range(args.warmup):
@@ -313,6 +334,8 @@ def compare_designs(args) -> int:
                      num_attention_heads=width // 128, num_key_value_heads=max(1, width // 512), tie_word_embeddings=True)
         if args.design == "zogurax":
             other = zogurax_config(width, layers, vocab, ff)
+        elif args.design == "peponex":
+            other = peponex_config(width, layers, vocab, ff)
         elif args.design == "zasidra":
             other = zasidra_config(width, layers, vocab, ff)
         elif args.design == "batodra":
@@ -321,7 +344,7 @@ def compare_designs(args) -> int:
             # two matrices a feed-forward instead of three: half as wide again for the same weight
             other = nipulorn_config(width, layers, vocab, ff * 3 // 2)
         entry = {"size": name, "layers": layers, args.design: measure(f"{args.design} {name}", other, vocab)}
-        if args.design == "batodra":
+        if args.design in ("batodra", "peponex"):
             # the other design that mixes recurrent layers with attention, at the same sizes
             entry["nipulorn"] = measure(f"nipulorn {name}", nipulorn_config(width, layers, vocab, ff * 3 // 2), vocab)
         if args.design == "zasidra":
@@ -335,7 +358,7 @@ def compare_designs(args) -> int:
 
 def main(argv=None) -> int:
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["nipulorn", "zogurax", "batodra", "zasidra"], default=None,
+    ap.add_argument("--design", choices=["nipulorn", "zogurax", "batodra", "zasidra", "peponex"], default=None,
                     help="instead of the default run: this design beside the dense decoder at equal sizes (prefill, decode, parts)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=248)   # + 8 warm-up = 256 new tokens

@@ -14,7 +14,7 @@
 // cs [T, rot_dims / 2] of (cos, sin), the rest pass unchanged; pairing 0: dimension i with
 // i + rot_dims / 2, pairing 1: neighbours (2i, 2i + 1).
 // qfull [T, ldq] float holds per head [dim | rot]; the head's rot part is rotated the same way
-// and written to q_out[t, h, rank .. rank + rot), zeros behind it up to hd.
+// and written to q_out[t, h, rank .. rank + rot), zeros behind it up to hd (n_heads 0: there are no queries).
 // With a value pool (the matrix cores' attention reads values in their own operand order) the
 // latent is stored there too, as dimensions 0..rank-1 of the token's value row.  With c_out the normed latents are
 // also left as plain rows [T, rank] (for a caller that multiplies them with the heads' key and value matrices).
@@ -70,7 +70,7 @@ LLOGOS_EXPORT int llogos_latent_prepare(const float* kv, int ldkv, const float* 
                                         const int* table, int table_stride, const int* tok_seq, const int* tok_pos,
                                         int T, int n_heads, int dim, int rot, int rot_dims, int pairing, int rank, int hd, void* c_out,
                                         hipStream_t stream) {
-    if (T <= 0 || n_heads <= 0 || dim < 0 || rot < 0 || rank <= 0 || hd < rank + rot || hd % 16) return LLOGOS_BAD_ARGUMENT;
+    if (T <= 0 || n_heads < 0 || dim < 0 || rot < 0 || rank <= 0 || hd < rank + rot || hd % 16) return LLOGOS_BAD_ARGUMENT;
     if (rot_dims < 0 || rot_dims > rot || rot_dims % 2 || (pairing != 0 && pairing != 1) || ldkv < rank + rot || ldq < n_heads * (dim + rot)) return LLOGOS_BAD_ARGUMENT;
     PagedKV cache{table, table_stride, 1, hd};
     if (dtype == DT_F32)

@@ -23,17 +23,12 @@ __global__ __launch_bounds__(1024) void qkv_prepare_kernel(
         const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w, float eps, float temp_coef, int temp_every,
         const float2* __restrict__ cs, int rot, int pairing,
         T* __restrict__ k_pool, T* __restrict__ v_pool, const int* __restrict__ table, int table_stride,
-        const int* __restrict__ tok_seq, const int* __restrict__ tok_pos, int staged_values,
-        const float* __restrict__ kv_rows, int kv_stride) {
+        const int* __restrict__ tok_seq, const int* __restrict__ tok_pos, int staged_values) {
     __shared__ float red[16];
     const int t = blockIdx.x, tid = threadIdx.x;
     const int Wq = n_heads * head_dim, Wk = n_kv_heads * head_dim, Wv = n_kv_heads * v_dim;
     const float* row = qkv + (size_t)t * row_stride;
     auto value = [&](int c) {
-        if (kv_rows && c >= Wq) {                            // keys and values that come in rows of their own
-            const float v = kv_rows[(size_t)t * kv_stride + (c - Wq)];
-            return bias ? v + bias[c] : v;
-        }
         float v = row[c];
         for (int p0 = 1; p0 < parts; p0 += 8) {              // eight loads in flight, added in ascending order
             float y[8];
@@ -107,14 +102,13 @@ __global__ __launch_bounds__(1024) void qkv_prepare_kernel(
 // qkv: float32 rows [T, row_stride] (row_stride >= the three widths together), `parts` of them
 // part_stride apart; bias float32 [Wq + Wk + Wv] or null; q_norm_w [Wq], k_norm_w [Wk] or null.
 // cs: float32 [T, rot / 2, 2] (cos, sin) or null with rot 0.
-// kv_rows (or null): float32 rows [T, kv_stride] that hold [k | v] in one part; qkv then holds q alone.
 // n_kv_heads 0: the keys and values of these positions are another run's; only q is made.
 LLOGOS_EXPORT int llogos_qkv_prepare(const float* qkv, int parts, long long part_stride, int row_stride, const float* bias,
                                      void* q_out, int dtype, int n_heads, int n_kv_heads, int head_dim, int v_dim,
                                      int k_page_dim, int v_page_dim, const float* q_norm_w, const float* k_norm_w, float eps,
                                      float temp_coef, int temp_every, const float* cs, int rot, int pairing,
                                      void* k_pool, void* v_pool, const int* table,
-                                     int table_stride, const int* tok_seq, const int* tok_pos, const float* kv_rows, int kv_stride,
+                                     int table_stride, const int* tok_seq, const int* tok_pos,
                                      int T, hipStream_t stream) {
     if (T <= 0 || n_heads <= 0 || n_kv_heads < 0 || head_dim <= 0 || v_dim <= 0 || parts < 1) return LLOGOS_BAD_ARGUMENT;
     if (temp_coef != 0.f && temp_every < 1) return LLOGOS_BAD_ARGUMENT;
@@ -123,16 +117,14 @@ LLOGOS_EXPORT int llogos_qkv_prepare(const float* qkv, int parts, long long part
         if (!k_pool || !v_pool || !table) return LLOGOS_BAD_ARGUMENT;
         if (k_page_dim < head_dim || v_page_dim < v_dim || (k_page_dim % 8) || (v_page_dim % 16)) return LLOGOS_BAD_ARGUMENT;
     }
-    if (kv_rows) {
-        if (row_stride < n_heads * head_dim || kv_stride < n_kv_heads * (head_dim + v_dim)) return LLOGOS_BAD_ARGUMENT;
-    } else if (row_stride < n_heads * head_dim + n_kv_heads * (head_dim + v_dim)) return LLOGOS_BAD_ARGUMENT;
+    if (row_stride < n_heads * head_dim + n_kv_heads * (head_dim + v_dim)) return LLOGOS_BAD_ARGUMENT;
     // few rows: many threads a row, so that a row's loads are all in flight at once
     const int threads = T <= 64 ? 1024 : 256;
     const int qk_values = n_heads * head_dim + n_kv_heads * head_dim;
     const int staged_values = (size_t)qk_values * sizeof(float) <= 48 * 1024 ? qk_values : 0;
 #define PREP(T_) qkv_prepare_kernel<T_><<<T, threads, staged_values * sizeof(float), stream>>>(qkv, parts, (size_t)part_stride, row_stride, bias, (T_*)q_out, \
         n_heads, n_kv_heads, head_dim, v_dim, k_page_dim, v_page_dim, q_norm_w, k_norm_w, eps, temp_coef, temp_every, \
-        (const float2*)cs, rot, pairing, (T_*)k_pool, (T_*)v_pool, table, table_stride, tok_seq, tok_pos, staged_values, kv_rows, kv_stride)
+        (const float2*)cs, rot, pairing, (T_*)k_pool, (T_*)v_pool, table, table_stride, tok_seq, tok_pos, staged_values)
     if (dtype == DT_F32) PREP(float);
     else if (dtype == DT_BF16) PREP(bf16_t);
     else return LLOGOS_BAD_ARGUMENT;

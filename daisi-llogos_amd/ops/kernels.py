@@ -347,27 +347,21 @@ def qkv_prepare(ctx, qkv: torch.Tensor, bias: Optional[torch.Tensor], out_dtype:
                 head_dim: int, v_dim: int, q_norm_w: Optional[torch.Tensor], k_norm_w: Optional[torch.Tensor], eps: float,
                 temp_coef: float, temp_every: int, k_pool: Optional[torch.Tensor], v_pool: Optional[torch.Tensor],
                 table: Optional[torch.Tensor], writes: bool = True, cs: Optional[torch.Tensor] = None, rot: int = 0,
-                pairing: int = 0, kv_rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+                pairing: int = 0) -> torch.Tensor:
     """From projected rows [q | k | v | ...] (float32 [T, >= W] or partial sums [parts, T, >= W], plus `bias`
     [W], W = n_heads * head_dim + n_kv_heads * (head_dim + v_dim)): an RMS norm over the whole of q and of
     k where a weight is given ([n_heads * head_dim], [n_kv_heads * head_dim]), then the rotation of the first
     `rot` dimensions of every head of q and k by the table `cs` [T, rot / 2, 2] (pairing 0: dimension i with
     i + rot / 2, 1: 2i with 2i + 1), the query's factor 1 + temp_coef * ln(floor((pos + 1) / temp_every) + 1);
     q comes back [T, n_heads * head_dim] in `out_dtype`, k and v go to their pages.  writes False: only q is
-    made (the rows then need hold no more than q).  kv_rows: float32 [T, >= n_kv_heads * (head_dim + v_dim)] rows
-    [k | v] in one part, for keys and values that were not projected together with q (qkv then holds q alone)."""
+    made (the rows then need hold no more than q)."""
     _need(qkv.is_cuda and qkv.dtype == torch.float32 and qkv.stride(-1) == 1, "qkv_prepare: float32 rows on the GPU")
     _dev(bias, q_norm_w, k_norm_w, table, ctx.tok_seq, ctx.tok_pos)
     parts, part_stride = _parts(qkv)
     T = qkv.shape[-2]
     Wq, Wk, Wv = n_heads * head_dim, n_kv_heads * head_dim, n_kv_heads * v_dim
-    width = Wq + ((Wk + Wv) if (writes and kv_rows is None) else 0)
+    width = Wq + ((Wk + Wv) if writes else 0)
     _need(qkv.shape[-1] >= width and T == ctx.n_tokens, f"qkv_prepare: rows of at least {width} values, one a token")
-    kv_stride = 0
-    if kv_rows is not None:
-        _need(writes and kv_rows.is_cuda and kv_rows.dtype == torch.float32 and kv_rows.dim() == 2 and kv_rows.shape[0] == T
-              and kv_rows.shape[1] >= Wk + Wv and kv_rows.stride(1) == 1, f"qkv_prepare: kv_rows must be float32 [T, >= {Wk + Wv}]")
-        kv_stride = kv_rows.stride(0) if T > 1 else max(Wk + Wv, kv_rows.stride(0))
     _need(rot % 2 == 0 and 0 <= rot <= head_dim and pairing in (0, 1), "qkv_prepare: the rotated width must be even and within a head")
     if rot:
         _dev(cs)
@@ -393,7 +387,7 @@ def qkv_prepare(ctx, qkv: torch.Tensor, bias: Optional[torch.Tensor], out_dtype:
         n_kv_heads if writes else 0, head_dim, v_dim, kd, vd, _p(q_norm_w), _p(k_norm_w), ctypes.c_float(eps),
         ctypes.c_float(temp_coef), int(temp_every), _p(cs) if rot else None, int(rot), int(pairing), _p(k_pool) if writes else None, _p(v_pool) if writes else None,
         _p(table) if writes else None, table.stride(0) if (writes and table is not None) else 0, _p(ctx.tok_seq), _p(ctx.tok_pos),
-        _p(kv_rows), kv_stride, T, _stream()), "qkv_prepare")
+        T, _stream()), "qkv_prepare")
     return q_out
 
 
@@ -770,30 +764,34 @@ def moe_combine(y: torch.Tensor, where: torch.Tensor, top: int, shared: Optional
 # ----------------------------------------------------------------------------
 # attention through a latent
 # ----------------------------------------------------------------------------
-def latent_prepare(ctx, kv: torch.Tensor, qfull: torch.Tensor, q_out: torch.Tensor, norm_w: torch.Tensor, eps: float,
+def latent_prepare(ctx, kv: torch.Tensor, qfull: Optional[torch.Tensor], q_out: Optional[torch.Tensor], norm_w: torch.Tensor, eps: float,
                    cs: Optional[torch.Tensor], k_pool: torch.Tensor, v_pool: Optional[torch.Tensor], table: torch.Tensor,
                    n_heads: int, dim: int, rot: int, rot_dims: int, rank: int, c_out: Optional[torch.Tensor] = None,
                    pairing: int = 1) -> None:
     """From kv float32 [T, rank + rot] and qfull float32 [T, heads * (dim + rot)]: the normed latent and
     the rotated shared key part go to the token's key row in the cache ([rank | rot | zeros]); each
-    head's rotated query part goes to q_out[t, h, rank:] ([T, heads, hd], hd the cache's row width).  With a
-    value pool the latent is also stored as the token's value row, and with c_out ([T, rank] of the cache's type)
-    as plain rows.  pairing 0: rotated dimension i is paired with i + rot_dims / 2, 1: 2i with 2i + 1."""
+    head's rotated query part goes to q_out[t, h, rank:] ([T, heads, hd], hd the cache's row width; qfull and q_out
+    None: no queries).  With a value pool the latent is also stored as the token's value row, and with c_out ([T, rank]
+    of the cache's type) as plain rows.  pairing 0: rotated dimension i is paired with i + rot_dims / 2, 1: 2i with 2i + 1."""
     _dev(q_out, norm_w, cs, k_pool, v_pool, table, ctx.tok_seq, ctx.tok_pos)
     _i32(table, "table")
     T = ctx.n_tokens
-    hd = q_out.shape[-1]
+    hd = k_pool.shape[-1] // PAGE_TOKENS
     # (kv and qfull may be columns of wider rows)
     _need(kv.is_cuda and kv.dtype == torch.float32 and kv.shape == (T, rank + rot) and kv.stride(1) == 1,
           "latent_prepare: kv must be float32 [T, rank + rot]")
-    _need(qfull.is_cuda and qfull.dtype == torch.float32 and qfull.shape == (T, n_heads * (dim + rot)) and qfull.stride(1) == 1,
-          "latent_prepare: q must be float32 [T, heads * (dim + rot)]")
-    _need(q_out.shape == (T, n_heads, hd) and q_out.dtype == k_pool.dtype, "latent_prepare: q_out must be [T, heads, hd] of the cache's type")
+    _need((qfull is None) == (q_out is None), "latent_prepare: queries and where they go, or neither")
+    if qfull is None:
+        n_heads = 0
+    else:
+        _need(qfull.is_cuda and qfull.dtype == torch.float32 and qfull.shape == (T, n_heads * (dim + rot)) and qfull.stride(1) == 1,
+              "latent_prepare: q must be float32 [T, heads * (dim + rot)]")
+        _need(q_out.shape == (T, n_heads, hd) and q_out.dtype == k_pool.dtype, "latent_prepare: q_out must be [T, heads, hd] of the cache's type")
     _need(hd % 16 == 0 and hd >= rank + rot, "latent_prepare: the cache's row is too narrow")
     _check_pools(k_pool, v_pool, 1, hd, "latent_prepare")
     _need(v_pool is None or v_pool.dtype == k_pool.dtype, "latent_prepare: the pools' types differ")
     _need(norm_w.dtype == torch.float32 and norm_w.shape == (rank,), "latent_prepare: norm weight must be float32 [rank]")
-    _need(rot_dims % 2 == 0 and 0 <= rot_dims <= rot, "latent_prepare: rotated dimensions must be even and within rot")
+    _need(rot_dims % 2 == 0 and 0 <= rot_dims <= rot and pairing in (0, 1), "latent_prepare: rotated dimensions must be even and within rot")
     if rot_dims:
         _need(cs is not None and cs.dtype == torch.float32 and cs.shape == (T, rot_dims // 2, 2), "latent_prepare: rotary table shape")
     _need(table.dim() == 2, "latent_prepare: page table must be [batch, pages]")
@@ -801,9 +799,40 @@ def latent_prepare(ctx, kv: torch.Tensor, qfull: torch.Tensor, q_out: torch.Tens
         _dev(c_out)
         _need(c_out.shape == (T, rank) and c_out.dtype == k_pool.dtype, "latent_prepare: c_out must be [T, rank] of the cache's type")
     ld = lambda t_, least: t_.stride(0) if T > 1 else max(least, t_.stride(0))
-    _check(_lib().llogos_latent_prepare(_p(kv), ld(kv, rank + rot), _p(qfull), ld(qfull, n_heads * (dim + rot)), _p(q_out), _dt(q_out), _p(norm_w),
-                                        ctypes.c_float(eps), _p(cs), _p(k_pool), _p(v_pool), _p(table), table.stride(0), _p(ctx.tok_seq),
-                                        _p(ctx.tok_pos), T, n_heads, dim, rot, rot_dims, int(pairing), rank, hd, _p(c_out), _stream()), "latent_prepare")
+    _check(_lib().llogos_latent_prepare(_p(kv), ld(kv, rank + rot), _p(qfull), ld(qfull, n_heads * (dim + rot)) if qfull is not None else 0,
+                                        _p(q_out), _dt(k_pool), _p(norm_w), ctypes.c_float(eps), _p(cs), _p(k_pool), _p(v_pool), _p(table),
+                                        table.stride(0), _p(ctx.tok_seq), _p(ctx.tok_pos), T, n_heads, dim, rot, rot_dims, int(pairing), rank,
+                                        hd, _p(c_out), _stream()), "latent_prepare")
+
+
+def latent_heads(ctx, kvh: torch.Tensor, kv: torch.Tensor, rank: int, q: torch.Tensor, cs: Optional[torch.Tensor], k_pool: torch.Tensor,
+                 v_pool: torch.Tensor, table: torch.Tensor, n_heads: int, dim: int, rot: int, rot_dims: int, pairing: int, v_dim: int) -> torch.Tensor:
+    """Keys, values and queries a head for a step of whole prompts (bfloat16): kvh [T, heads * dim + heads * v_dim] holds
+    every head's unrotated keys and then its values, kv float32 [T, >= rank + rot] the shared key part behind `rank`
+    values, q float32 [T, heads * (dim + rot)].  Keys [dim | rotated part] and values go to the pages of `table`
+    (pools [pages, heads, 64 * (dim + rot)] and [pages, heads, 64 * v_dim]); the queries come back [T, heads * (dim + rot)]."""
+    _dev(kvh, cs, k_pool, v_pool, table, ctx.cu_dev)
+    _i32(table, "table")
+    T, dk = ctx.n_tokens, dim + rot
+    _need(kvh.dtype == torch.bfloat16 and kvh.shape == (T, n_heads * (dim + v_dim)), "latent_heads: kvh must be bfloat16 [T, heads * (dim + v_dim)]")
+    _need(kv.is_cuda and kv.dtype == torch.float32 and kv.dim() == 2 and kv.shape[0] == T and kv.shape[1] >= rank + rot and kv.stride(1) == 1,
+          "latent_heads: kv must be float32 [T, rank + rot]")
+    _need(q.is_cuda and q.dtype == torch.float32 and q.shape == (T, n_heads * dk) and q.stride(1) == 1, "latent_heads: q must be float32 [T, heads * (dim + rot)]")
+    _need(dim % 8 == 0 and rot % 8 == 0 and dk % 16 == 0 and v_dim % 16 == 0, "latent_heads: widths must be multiples of 8, of values 16")
+    _need(rot_dims % 2 == 0 and 0 <= rot_dims <= rot and pairing in (0, 1), "latent_heads: rotated dimensions must be even and within rot")
+    if rot_dims:
+        _need(cs is not None and cs.dtype == torch.float32 and cs.shape == (T, rot_dims // 2, 2), "latent_heads: rotary table shape")
+    _need(k_pool.dtype == torch.bfloat16 and v_pool.dtype == torch.bfloat16 and k_pool.shape[0] == v_pool.shape[0]
+          and tuple(k_pool.shape[1:]) == (n_heads, PAGE_TOKENS * dk) and tuple(v_pool.shape[1:]) == (n_heads, PAGE_TOKENS * v_dim),
+          "latent_heads: pools [pages, heads, 64 * width]")
+    n_pages = sum(-(-(ctx.cu_seqlens[i + 1] - ctx.cu_seqlens[i]) // PAGE_TOKENS) for i in range(ctx.batch))
+    _need(table.dim() == 2 and table.shape[0] == ctx.batch and k_pool.shape[0] >= n_pages and ctx.cu_dev is not None, "latent_heads: a page for every 64 tokens")
+    q_out = torch.empty((T, n_heads * dk), dtype=torch.bfloat16, device=q.device)
+    ld = lambda t_, least: t_.stride(0) if T > 1 else max(least, t_.stride(0))
+    _check(_lib().llogos_latent_heads(_p(kvh), _p(kv), ld(kv, rank + rot), rank, _p(q), ld(q, n_heads * dk), _p(cs) if rot_dims else None, _p(q_out),
+                                      _p(k_pool), _p(v_pool), _p(table), table.stride(0), _p(ctx.cu_dev), ctx.batch, n_pages, n_heads, dim, rot,
+                                      rot_dims, int(pairing), v_dim, _stream()), "latent_heads")
+    return q_out
 
 
 LATENT_MFMA_MAX_ROW = 576
@@ -2041,12 +2070,13 @@ CAPPED_PREFILL_HALVES = 0         # 0: chosen by the step; 1 or 2 sets of waves 
 
 def capped_attention(ctx, q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, table: torch.Tensor, n_heads: int,
                      n_kv_heads: int, head_dim: int, v_dim: int, scale: float, softcap: float = 0.0,
-                     head_sink: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     head_sink: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, window: int = 0) -> torch.Tensor:
     """Causal attention of the step's query rows q [T, n_heads * head_dim] over their sequences' pages, for keys of
     head_dim and values of v_dim dimensions: scores bent to softcap * tanh(score / softcap) (softcap > 0), a sink in
     the softmax's denominator (head_sink float32 [n_heads]: exp(head_sink[h]) is added to head h's sums; zeros for a
     sink of score 0), head h's output times
-    sigmoid(gate[t, h]) (gate float32 [T, >= n_heads], maybe a view of wider rows).  Returns [T, n_heads * v_dim].
+    sigmoid(gate[t, h]) (gate float32 [T, >= n_heads], maybe a view of wider rows); window > 0: a query sees the last
+    `window` keys, its own among them.  Returns [T, n_heads * v_dim].
     bfloat16 with head sizes the matrix-core kernels take runs there; everything else in the kernel for any shape."""
     T = ctx.n_tokens
     if q.dtype == torch.bfloat16 and q.dim() == 2 and q.is_contiguous():
@@ -2065,7 +2095,9 @@ def capped_attention(ctx, q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
             if head_sink is not None:
                 _dev(head_sink)
                 _need(head_sink.dtype == torch.float32 and head_sink.shape == (n_heads,), "attention: head_sink must be float32 [n_heads]")
-            if ctx.is_decode:
+            if ctx.is_decode and window > 0:
+                code = -2
+            elif ctx.is_decode:
                 width = table.shape[1]
                 _need(table.shape[0] == T and ctx.tok_pos.numel() == T, "attention: one table row and position a sequence")
                 ws = _attn_workspace(q.device, lib.llogos_capped_attn_decode_workspace(T, n_heads, n_kv_heads, v_dim, width))
@@ -2079,10 +2111,15 @@ def capped_attention(ctx, q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
                 # long sequences: tiles of 128 tokens whose pages go straight into LDS once for a block's waves (the
                 # dense decoder's prompt kernel with the bent softmax); short ones: tiles of 64 whose waves read the pages
                 lens = [ctx.cu_seqlens[i + 1] - ctx.cu_seqlens[i] for i in range(ctx.batch)]
-                tile_rows = CAPPED_PREFILL_TILE_ROWS or (128 if max(lens) > 64 else 64)
+                # (a window, or keys of 192 dimensions, in the 128-row form alone)
+                wide = window > 0 or head_dim == 192
+                tile_rows = 128 if wide else (CAPPED_PREFILL_TILE_ROWS or (128 if max(lens) > 64 else 64))
                 n_tiles = sum(-(-n // tile_rows) for n in lens)
                 halves = CAPPED_PREFILL_HALVES or (prefill_halves(lens, getattr(ctx, "starts", None), n_heads) if tile_rows == 128 else 1)
-                code = lib.llogos_capped_attn_prefill_bf16(
+                code = lib.llogos_wide_attn_prefill_bf16(
+                    _p(out), _p(q), q.stride(0), _p(k_pool), _p(v_pool), _p(table), table.stride(0), _p(cu), _p(ctx.tok_pos),
+                    ctx.batch, n_tiles, n_heads, n_kv_heads, head_dim, v_dim, ctypes.c_float(scale), int(window), _p(head_sink), _p(gate),
+                    gate_stride, int(halves), _stream()) if wide and softcap == 0.0 else -2 if wide else lib.llogos_capped_attn_prefill_bf16(
                     _p(out), _p(q), q.stride(0), _p(k_pool), _p(v_pool), _p(table), table.stride(0), _p(cu), _p(ctx.tok_pos),
                     ctx.batch, n_tiles, n_heads, n_kv_heads, head_dim, v_dim, ctypes.c_float(scale), ctypes.c_float(softcap),
                     _p(head_sink), _p(gate), gate_stride, int(tile_rows), int(halves), _stream())
@@ -2090,7 +2127,7 @@ def capped_attention(ctx, q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
                 _check(code, "capped_attention")
                 return out
     return attention_generic(q, n_heads * head_dim, k_pool, v_pool, table, ctx.tok_seq, ctx.tok_pos, n_heads, n_kv_heads,
-                             head_dim, scale, v_dim=v_dim, head_sink=head_sink, softcap=softcap, gate=gate)
+                             head_dim, scale, window=window, v_dim=v_dim, head_sink=head_sink, softcap=softcap, gate=gate)
 
 
 # ----------------------------------------------------------------------------

@@ -15,10 +15,10 @@ head's query becomes [W_uk,h^T q_h,plain | q_h,rot] against the cached row, the 
 over latents, and W_uv,h is applied to that sum (the gate in that product's epilogue).  The
 projections that read h (q or dq, dkv, g) are one stacked product.
 
-Whole prompts in bfloat16 whose head shapes the matrix cores' attention takes, and that have no rotated
-part, go the other way round: the step's latents are multiplied with all heads' key and value matrices at
-once (one product of the library's kind), the keys and values go to pages of the step's own, and the
-prompt kernel of the attention with keys and values a head runs on them: a quarter or less of the
+Whole prompts in bfloat16 whose head shapes the matrix cores' attention takes go the other way round: the
+step's latents are multiplied with all heads' key and value matrices at once (one product of the library's
+kind), the keys (with the rotated part behind every head's own) and values go to pages of the step's own, and
+the prompt kernel of the attention with keys and values a head runs on them: a quarter or less of the
 arithmetic of scores and sums over latents, on the faster kernel.  The cache still gets the latents alone."""
 from __future__ import annotations
 
@@ -124,8 +124,8 @@ class LatentAttention(Mixer):
 
     def _heads_on_matrix_cores(self) -> bool:
         """Whether whole prompts can run as attention with keys and values a head (see the module's text)."""
-        return self.rt.dtype == torch.bfloat16 and self.rot_dim == 0 and self.window == 0 and not self.q_rank and self.dim in (64, 96, 128) \
-            and self.v_dim in (64, 80, 96, 128)
+        return self.rt.dtype == torch.bfloat16 and self.dim + self.rot_dim in (64, 96, 128, 192) and self.v_dim in (64, 80, 96, 128) \
+            and self.dim % 8 == 0 and self.rot_dim % 8 == 0 and not (self.window and (self.has_sink or self.head_gate))
 
     @staticmethod
     def _prompt_pages(ctx: StepContext):
@@ -148,21 +148,26 @@ class LatentAttention(Mixer):
         mark(ctx, "o")
         return out
 
-    def _forward_prompt(self, ctx: StepContext, rows: torch.Tensor, kv: torch.Tensor, gate, cache: LayerCache,
+    def _rotation(self, ctx: StepContext):
+        """(table of cosines and sines or None, rotated dimensions, pairing) for this step."""
+        if self.position is None:
+            return None, 0, 1
+        return self.position.prepare(ctx), self.position.rot, self.position.pairing
+
+    def _forward_prompt(self, ctx: StepContext, kv: torch.Tensor, q: torch.Tensor, gate, cache: LayerCache,
                         residual: Optional[Residual]):
-        f32, H, T = torch.float32, self.n_heads, ctx.n_tokens
-        qa = torch.empty((T, H, self.row), dtype=self.rt.dtype, device=rows.device)       # (no rotated part: nothing is written)
-        c = torch.empty((T, self.kv_rank), dtype=self.rt.dtype, device=rows.device)
-        K.latent_prepare(ctx, kv, rows[:, :self.q_width], qa, self.c_norm_w, self.eps, None, cache.k_pool, cache.v_pool, cache.table,
-                         H, self.dim, 0, 0, self.kv_rank, c_out=c)
-        keys_values = K.sum_parts(K.gemm_product(c, self.ukv, self.rt.dtype, f32_ok=True), None, f32)     # [T, H * (dim + v_dim)]
-        mark(ctx, "rotation")
+        H, T, dk = self.n_heads, ctx.n_tokens, self.dim + self.rot_dim
+        cs, rot_dims, pairing = self._rotation(ctx)
+        c = torch.empty((T, self.kv_rank), dtype=self.rt.dtype, device=kv.device)
+        K.latent_prepare(ctx, kv, None, None, self.c_norm_w, self.eps, cs, cache.k_pool, cache.v_pool, cache.table, 0, self.dim, self.rot_dim,
+                         rot_dims, self.kv_rank, c_out=c, pairing=pairing)
+        kvh = K.sum_parts(K.gemm_product(c, self.ukv, self.rt.dtype), None, self.rt.dtype)                # [T, H * (dim + v_dim)]
         n_pages, table = self._prompt_pages(ctx)
-        k_pool = torch.empty((n_pages, H, K.PAGE_TOKENS * self.dim), dtype=self.rt.dtype, device=rows.device)
-        v_pool = torch.empty((n_pages, H, K.PAGE_TOKENS * self.v_dim), dtype=self.rt.dtype, device=rows.device)
-        q = K.qkv_prepare(ctx, rows, None, self.rt.dtype, H, H, self.dim, self.v_dim, None, None, self.eps, 0.0, 1, k_pool, v_pool,
-                          table, kv_rows=keys_values)
-        a = K.capped_attention(ctx, q, k_pool, v_pool, table, H, H, self.dim, self.v_dim, self.scale, 0.0, self.sink, gate)
+        k_pool = torch.empty((n_pages, H, K.PAGE_TOKENS * dk), dtype=self.rt.dtype, device=kv.device)
+        v_pool = torch.empty((n_pages, H, K.PAGE_TOKENS * self.v_dim), dtype=self.rt.dtype, device=kv.device)
+        qh = K.latent_heads(ctx, kvh, kv, self.kv_rank, q, cs, k_pool, v_pool, table, H, self.dim, self.rot_dim, rot_dims, pairing, self.v_dim)
+        mark(ctx, "rotation")
+        a = K.capped_attention(ctx, qh, k_pool, v_pool, table, H, H, dk, self.v_dim, self.scale, 0.0, self.sink, gate, self.window)
         mark(ctx, "attention")
         return self._close(ctx, a, residual)
 
@@ -181,12 +186,11 @@ class LatentAttention(Mixer):
         mark(ctx, "projections")
         if self.ukv is not None and not ctx.is_decode and not ctx.in_graph and T >= self.prompt_rows and ctx.cu_dev is not None \
                 and not any(ctx.starts):
-            return self._forward_prompt(ctx, rows, kv, gate, cache, residual)
-        cs = self.position.prepare(ctx) if self.position is not None else None
+            return self._forward_prompt(ctx, kv, q, gate, cache, residual)
+        cs, rot_dims, pairing = self._rotation(ctx)
         qa = torch.empty((T, H, self.row), dtype=self.rt.dtype, device=h.device)
         K.latent_prepare(ctx, kv, q, qa, self.c_norm_w, self.eps, cs, cache.k_pool, cache.v_pool, cache.table, H, self.dim, self.rot_dim,
-                         self.position.rot if self.position is not None else 0, self.kv_rank,
-                         pairing=self.position.pairing if self.position is not None else 1)
+                         rot_dims, self.kv_rank, pairing=pairing)
         K.head_products(q.unflatten(1, (H, self.dim + self.rot_dim))[:, :, :self.dim], self.uk_t, qa[:, :, :self.kv_rank], self.uk_kn)
         mark(ctx, "rotation")
         lat = None
