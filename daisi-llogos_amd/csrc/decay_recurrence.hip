@@ -130,7 +130,7 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(float* __restrict__ o,
                                                           size_t part_stride, const float* __restrict__ powers,
                                                           float* __restrict__ state, size_t state_stride, const int* __restrict__ slots,
                                                           const int* __restrict__ cu, int H, int D, int V, int col_blocks, int n_seg,
-                                                          int seg_len, float* __restrict__ seg_state) {
+                                                          int seg_len, float* __restrict__ seg_state, int vec) {
     constexpr int C = kDecayChunk, DP = 16 * DT + kDecayPad, CP = C + kDecayPad, VB = 64 * VT;
     extern __shared__ __attribute__((aligned(16))) float lds[];
     float* sQ = lds;                       // [C][DP]   rows times a^(i + 1) where the state is read: the factor comes with the store of o
@@ -160,28 +160,53 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(float* __restrict__ o,
                 const int d = 16 * dt + 4 * g + r, col = col0 + 16 * vt + c;
                 s[dt][vt][r] = (MODE != 1 && d < D && col < V) ? S[(size_t)d * V + col] : 0.f;
             }
-    auto value = [&](const float* p) {
-        float z = *p;
-        for (int q = 1; q < parts; ++q) z += p[q * part_stride];
-        return decay_silu(z);
+    // four neighbouring values of a token's row, from column `at` on (those at or behind `end` are zeros), activated
+    auto value4 = [&](int j, int n, size_t at, size_t end) {
+        float4 z = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (j < n && at < end) {
+            const float* p = rows + (size_t)(first + j) * ld + at;
+            for (int q = 0; q < parts; ++q, p += part_stride) {
+                if (vec) {
+                    const float4 u = *reinterpret_cast<const float4*>(p);
+                    z.x += u.x; z.y += u.y; z.z += u.z; z.w += u.w;
+                } else {
+                    z.x += p[0];
+                    if (at + 1 < end) z.y += p[1];
+                    if (at + 2 < end) z.z += p[2];
+                    if (at + 3 < end) z.w += p[3];
+                }
+            }
+            z = make_float4(decay_silu(z.x), decay_silu(z.y), decay_silu(z.z), decay_silu(z.w));
+        }
+        return z;
     };
     for (int t0 = 0; t0 < count; t0 += C) {
         const int n = min(C, count - t0);
         __syncthreads();                                   // the chunk before has been read (and pw is there)
-        for (int e = tid; e < C * 16 * DT; e += 256) {
-            const int j = e / (16 * DT), d = e % (16 * DT);
-            float q = 0.f, k = 0.f;
-            if (j < n && d < D) {
-                const float* row = rows + (size_t)(first + t0 + j) * ld;
-                k = value(row + (size_t)(H + head) * D + d);
-                if (MODE != 1) q = value(row + (size_t)head * D + d);
+        // (a wave takes 16 rows, 64 bytes of each: the transposed copies' stores then fall on neighbouring words of a row)
+#pragma unroll 4
+        for (int e = tid; e < C * 4 * DT; e += 256) {
+            const int j = (e & 15) + 16 * ((e >> 4) / (4 * DT)), d = 4 * ((e >> 4) % (4 * DT));
+            const float4 k = value4(t0 + j, t0 + n, (size_t)(H + head) * D + d, (size_t)(H + head + 1) * D);
+            if (MODE != 1) {
+                *reinterpret_cast<float4*>(sQ + j * DP + d) = value4(t0 + j, t0 + n, (size_t)head * D + d, (size_t)(head + 1) * D);
+                *reinterpret_cast<float4*>(sK + j * DP + d) = k;
             }
-            if (MODE != 1) { sQ[j * DP + d] = q; sK[j * DP + d] = k; }
-            sKT[d * CP + j] = j < n ? k * pw[n - 1 - j] : 0.f;
+            const float f = j < n ? pw[n - 1 - j] : 0.f;
+            sKT[(d + 0) * CP + j] = k.x * f;
+            sKT[(d + 1) * CP + j] = k.y * f;
+            sKT[(d + 2) * CP + j] = k.z * f;
+            sKT[(d + 3) * CP + j] = k.w * f;
         }
-        for (int e = tid; e < C * VB; e += 256) {
-            const int j = e / VB, i = e % VB, col = cb * VB + i;
-            sVT[i * CP + j] = (j < n && col < V) ? value(rows + (size_t)(first + t0 + j) * ld + (size_t)2 * H * D + (size_t)head * V + col) : 0.f;
+#pragma unroll 4
+        for (int e = tid; e < C * VB / 4; e += 256) {
+            const int j = (e & 15) + 16 * ((e >> 4) / (VB / 4)), i = 4 * ((e >> 4) % (VB / 4));
+            const size_t v0 = (size_t)2 * H * D + (size_t)head * V;
+            const float4 v = value4(t0 + j, t0 + n, v0 + cb * VB + i, v0 + V);
+            sVT[(i + 0) * CP + j] = v.x;
+            sVT[(i + 1) * CP + j] = v.y;
+            sVT[(i + 2) * CP + j] = v.z;
+            sVT[(i + 3) * CP + j] = v.w;
         }
         __syncthreads();
         if (MODE != 1) {
@@ -356,6 +381,7 @@ LLOGOS_EXPORT int llogos_decay_scan(float* o, const float* rows, int ld, int par
     const int dt = (D + 15) / 16, vt = V > 64 ? 2 : 1;
     const int col_blocks = (V + 64 * vt - 1) / (64 * vt);
     dim3 grid(B, H, col_blocks * n_seg);
+    const int vec4 = D % 4 == 0 && V % 4 == 0 && ld % 4 == 0 && part_stride % 4 == 0 && (uintptr_t)rows % 16 == 0 ? 1 : 0;
 #define DC(DT, VT, MODE) do { \
         const int smem = decay_lds_floats(DT, VT) * (int)sizeof(float); \
         if (smem > 48 * 1024) { \
@@ -363,7 +389,7 @@ LLOGOS_EXPORT int llogos_decay_scan(float* o, const float* rows, int ld, int par
             if (e != hipSuccess) return (int)e; \
         } \
         decay_chunk_kernel<DT, VT, MODE><<<grid, 256, smem, stream>>>(o, rows, ld, parts, (size_t)part_stride, powers, state, \
-            (size_t)state_stride, slots, cu, H, D, V, col_blocks, n_seg, seg_len, seg_state); } while (0)
+            (size_t)state_stride, slots, cu, H, D, V, col_blocks, n_seg, seg_len, seg_state, vec4); } while (0)
 #define DCM(DT, VT) do { \
         if (n_seg == 1) { DC(DT, VT, 0); break; } \
         DC(DT, VT, 1); \
