@@ -784,7 +784,7 @@ def _drawn(seed: int) -> dict:
     """A configuration drawn from a seed over everything the file can vary."""
     rng = np.random.default_rng(seed)
     pick = lambda *xs: xs[int(rng.integers(len(xs)))]
-    W = int(pick(40, 48, 64, 72, 96))
+    W = int(pick(40, 48, 64, 72, 96)) if seed < 16 else int(pick(50, 100))          # (widths that no vector load divides, too)
     layers = []
     for i in range(int(rng.integers(2, 6))):
         mlp = None
@@ -815,7 +815,7 @@ def _drawn(seed: int) -> dict:
     return cfg
 
 
-@pytest.mark.parametrize("seed", range(16))
+@pytest.mark.parametrize("seed", range(20))
 def test_configurations_drawn_from_seeds(seed, tmp_path):
     """Ragged prompts, single tokens, a sequence that ends early and a new prompt in the freed slot beside one that goes on."""
     from safetensors.torch import load_file, save_file
