@@ -100,3 +100,12 @@ def _peponex() -> None:
 
 
 _peponex()
+
+
+def _zisedra() -> None:
+    from ..models.zisedra import zisedra_spec
+    from .zisedra_config import ZisedraConfig
+    register_architecture("Zisedra", ZisedraConfig.from_dict, zisedra_spec, reads_shapes=True)
+
+
+_zisedra()

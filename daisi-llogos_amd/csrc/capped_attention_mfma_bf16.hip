@@ -1,7 +1,8 @@
 // bfloat16 attention on the matrix cores for heads whose keys and values have different widths,
 // whose scores may be bent through a tanh (s -> cap * tanh(s / cap)), whose softmax may carry a
 // sink (a score a head without a key or a value: exp(sink) joins the denominator) and whose output may be gated head by head
-// (sigmoid of a logit a token and head).  No window: a query sees every key up to its own.
+// (sigmoid of a logit a token and head).  A query sees every key up to its own; single-token steps also take a window
+// (plain scores; a page that lies outside it is not read, since it may have been given back).
 //
 // Keys are rows of KP = 32 KS dimensions in their pages, values rows of VP = 16 VB; the pages are
 // in the matrix cores' operand order (common.h), so the page steps of attention_mfma.h serve:
@@ -19,7 +20,7 @@
 template <int KP, int VP>
 __device__ __forceinline__ void attend_page_kv(WaveState<VP>& st, const bf16x8 (&qf)[KP / 32], const bf16_t* __restrict__ kpage,
                                                const bf16_t* __restrict__ vpage, int q_pos, int key0, int valid_keys,
-                                               bool all_visible, float scale, float cap) {
+                                               bool all_visible, float scale, float cap, int window = 0) {
     bf16x8 kf[4][KP / 32], vf[VP / 16][2];
     load_keys<KP>(kf, kpage);
     load_values<VP>(vf, vpage);
@@ -27,8 +28,9 @@ __device__ __forceinline__ void attend_page_kv(WaveState<VP>& st, const bf16x8 (
     page_scores<KP>(s, kf, qf);
     bf16x8 pf[2];
     float corr;
-    if (all_visible) softmax_page_bent<false, VP>(s, st, scale, cap, q_pos, key0, pf, corr);
-    else             softmax_page_bent<true, VP>(s, st, scale, cap, q_pos, key0, pf, corr);
+    if (window > 0)       softmax_page<true, 16, 4, VP>(s, st, scale * kLog2e, q_pos, key0, window, 0, pf, corr);
+    else if (all_visible) softmax_page_bent<false, VP>(s, st, scale, cap, q_pos, key0, pf, corr);
+    else                  softmax_page_bent<true, VP>(s, st, scale, cap, q_pos, key0, pf, corr);
     weigh_values<VP>(st, vf, pf, corr, valid_keys);
 }
 
@@ -133,7 +135,7 @@ template <int KS, int VB>
 __global__ __launch_bounds__(kAttnWaves * kWave) void capped_decode_kernel(
         bf16_t* __restrict__ out, float* __restrict__ partial, const bf16_t* __restrict__ q, int q_stride,
         const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool, const int* __restrict__ table, int table_stride,
-        const int* __restrict__ tok_pos, int n_heads, int n_kv_heads, int group, float scale, float cap, int ppw,
+        const int* __restrict__ tok_pos, int n_heads, int n_kv_heads, int group, float scale, float cap, int window, int ppw,
         const float* __restrict__ head_sink, const float* __restrict__ gate, int gate_stride) {
     constexpr int KP = 32 * KS, VP = 16 * VB, WAVES = kAttnWaves;
     extern __shared__ float lds[];
@@ -160,9 +162,10 @@ __global__ __launch_bounds__(kAttnWaves * kWave) void capped_decode_kernel(
         const int pi = first_page + wave + WAVES * j;
         if (pi >= n_pages) break;
         const int key0 = pi * kPageTokens;
+        if (!page_may_be_visible(pos, key0, window, 0)) continue;
         const size_t page = ((size_t)row[pi] * n_kv_heads + kvh) * kPageTokens;
         attend_page_kv<KP, VP>(st, qf, k_pool + page * KP, v_pool + page * VP, col_ok ? pos : -1, key0,
-                               min(kPageTokens, pos - key0 + 1), key0 + kPageTokens - 1 <= pos, scale, cap);
+                               min(kPageTokens, pos - key0 + 1), key0 + kPageTokens - 1 <= pos, scale, cap, window);
     }
     if (g == 0) { lds_m[wave * 16 + c] = st.m; lds_l[wave * 16 + c] = st.l; }
     if (col_ok) {
@@ -309,9 +312,9 @@ LLOGOS_EXPORT long long llogos_capped_attn_decode_workspace(int batch, int n_hea
 LLOGOS_EXPORT int llogos_capped_attn_decode_bf16(void* out, const void* q, int q_stride, const void* k_pool, const void* v_pool,
                                                  const int* table, int table_stride, int table_width, const int* tok_pos,
                                                  int batch, int n_heads, int n_kv_heads, int dk, int dv, float scale,
-                                                 float softcap, const float* head_sink, const float* gate, int gate_stride,
+                                                 float softcap, int window, const float* head_sink, const float* gate, int gate_stride,
                                                  float* workspace, long long workspace_floats, hipStream_t stream) {
-    if (batch <= 0 || table_width <= 0 || softcap < 0.f || (gate && gate_stride < n_heads)) return LLOGOS_BAD_ARGUMENT;
+    if (batch <= 0 || table_width <= 0 || softcap < 0.f || window < 0 || (window > 0 && softcap > 0.f) || (gate && gate_stride < n_heads)) return LLOGOS_BAD_ARGUMENT;
     if (!capped_shape_ok(n_heads, n_kv_heads, dk, dv) || q_stride % 8) return LLOGOS_UNSUPPORTED;
     const int group = n_heads / n_kv_heads;
     const int ppw = capped_pages_per_wave(batch, n_kv_heads, table_width);
@@ -321,7 +324,7 @@ LLOGOS_EXPORT int llogos_capped_attn_decode_bf16(void* out, const void* q, int q
     const size_t lds = (size_t)kAttnWaves * (group * (dv + 1) + 32) * sizeof(float);
 #define DEC(KS, VB) capped_decode_kernel<KS, VB><<<grid, kAttnWaves * kWave, lds, stream>>>((bf16_t*)out, workspace, (const bf16_t*)q, \
         q_stride, (const bf16_t*)k_pool, (const bf16_t*)v_pool, table, table_stride, tok_pos, n_heads, n_kv_heads, group, scale, \
-        softcap, ppw, head_sink, gate, gate_stride)
+        softcap, window, ppw, head_sink, gate, gate_stride)
     CAPPED_SHAPES(DEC)
 #undef DEC
     if (n_z > 1) {

@@ -60,12 +60,20 @@ LLOGOS_EXPORT int llogos_moe_route(const int* ids, const int* table, int T, int 
     return LLOGOS_LAUNCH_CHECK();
 }
 
-__device__ __forceinline__ float moe_gated(float gate, float up) { return gate / (1.0f + expf(-gate)) * up; }
+// the two ways in which a gate and an up sum become one value: 2 silu(gate) * up; 3 with g = min(gate, limit) and
+// u = up kept within -limit .. limit, g * sigmoid(1.702 g) * (u + 1)
+__device__ __forceinline__ float moe_gated(float gate, float up, int act, float limit) {
+    if (act == 3) {
+        const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+        return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+    }
+    return gate / (1.0f + expf(-gate)) * up;
+}
 
 // out[r, :] = act(a_row(r) . w[e]^T) * scale for the sorted rows r of expert e's segment.
 // act 0: none; 1: the square of relu; 2: the matrix's rows are gate and up rows in turn (gate 0, up 0, gate 1, ...)
-// and the result has N / 2 columns silu(gate_i) * up_i.
-// With row_weight (act 2 only) a row's gate and up sums are multiplied by row_weight[order[r]] first: the product of the
+// and the result has N / 2 columns silu(gate_i) * up_i; 3: the same with both sums bounded by `limit` (moe_gated).
+// With row_weight (act 2 or 3 only) a row's gate and up sums are multiplied by row_weight[order[r]] first: the product of the
 // row times its pair's weight.
 // a_row(r) = a[order[r] / top] when gather (the step's token rows), else a[r] (rows already sorted).
 // w is [E][N][K].  Tiles of 64 rows x 64 columns; blockIdx.y counts row tiles over all segments.
@@ -75,7 +83,7 @@ template <typename TA, typename TW, typename TO>
 __global__ __launch_bounds__(256) void moe_product_kernel(TO* __restrict__ out, const TA* __restrict__ a, const TW* __restrict__ w,
                                                           const int* __restrict__ order, const int* __restrict__ seg, int E,
                                                           int top, int gather, int N, int K, int lda, int act, float scale,
-                                                          const float* __restrict__ row_weight) {
+                                                          const float* __restrict__ row_weight, float limit) {
     __shared__ float As[GK][GM + 4];
     __shared__ float Ws[GK][GN + 4];
     __shared__ int src_row[GM];
@@ -140,13 +148,13 @@ __global__ __launch_bounds__(256) void moe_product_kernel(TO* __restrict__ out, 
         const int m = m0 + ty * 4 + i;
         if (m >= m_end) continue;
         const float rw = row_weight ? row_weight[order[m]] : 1.0f;
-        if (act == 2) {                                     // columns in pairs (gate, up): silu(gate) * up
+        if (act >= 2) {                                     // columns in pairs (gate, up): silu(gate) * up
 #pragma unroll
             for (int j = 0; j < 4; j += 2) {
                 const int n = n0 + tx * 4 + j;
                 if (n + 1 >= N) continue;
                 const float gt = acc[i][j] + mid[i][j], up = acc[i][j + 1] + mid[i][j + 1];
-                store_f32(out + (size_t)m * (N / 2) + n / 2, moe_gated(gt * rw, up * rw) * scale);
+                store_f32(out + (size_t)m * (N / 2) + n / 2, moe_gated(gt * rw, up * rw, act, limit) * scale);
             }
             continue;
         }
@@ -164,13 +172,13 @@ __global__ __launch_bounds__(256) void moe_product_kernel(TO* __restrict__ out, 
 // P = T * top sorted rows at most; row_tiles bounds the tiles of all segments: ceil(P / 64) + E covers them.
 LLOGOS_EXPORT int llogos_moe_product(void* out, int out_dtype, const void* a, int a_dtype, const void* w, int w_dtype,
                                      const int* order, const int* seg, int E, int top, int gather, int P, int N, int K,
-                                     int lda, int act, float scale, const float* row_weight, hipStream_t stream) {
-    if (P <= 0 || N <= 0 || K <= 0 || E <= 0 || top <= 0 || lda < K || act < 0 || act > 2 || (act == 2 && (N & 1)) || (row_weight && act != 2)) return LLOGOS_BAD_ARGUMENT;
+                                     int lda, int act, float scale, const float* row_weight, float limit, hipStream_t stream) {
+    if (P <= 0 || N <= 0 || K <= 0 || E <= 0 || top <= 0 || lda < K || act < 0 || act > 3 || (act >= 2 && (N & 1)) || (row_weight && act < 2) || (act == 3 && !(limit >= 0.f))) return LLOGOS_BAD_ARGUMENT;
     if (a_dtype != w_dtype && !(a_dtype == DT_F32)) return LLOGOS_BAD_ARGUMENT;
     const int row_tiles = (P + GM - 1) / GM + E;
     dim3 grid((N + GN - 1) / GN, row_tiles);
 #define MP(TA, TW, TO) moe_product_kernel<TA, TW, TO><<<grid, 256, 0, stream>>>((TO*)out, (const TA*)a, (const TW*)w, order, seg, E, \
-        top, gather, N, K, lda, act, scale, row_weight)
+        top, gather, N, K, lda, act, scale, row_weight, limit)
     if (a_dtype == DT_F32 && w_dtype == DT_F32 && out_dtype == DT_F32) MP(float, float, float);
     else if (a_dtype == DT_BF16 && w_dtype == DT_BF16 && out_dtype == DT_BF16) MP(bf16_t, bf16_t, bf16_t);
     else if (a_dtype == DT_BF16 && w_dtype == DT_BF16 && out_dtype == DT_F32) MP(bf16_t, bf16_t, float);
@@ -323,14 +331,15 @@ __device__ __forceinline__ int wave_best_open(const float* v, const unsigned cha
 
 // One wave a token.  From the router's logits z [T, E] (float32):
 //   s = softmax(z) over all E outputs;  c = s + correction  (the choice's scores; correction may be null)
-//   the E outputs form n_groups equal groups of neighbours; a group's score is its largest c; outputs outside the
+//   the E outputs form n_groups equal groups of neighbours; a group's score is its largest c (group_best 1) or the sum
+//   of its two largest (2; of its only one where a group is a single output); outputs outside the
 //   `keep` best groups cannot be chosen (n_groups <= 1 or keep >= n_groups: all can)
 //   choice[t, j] = the j-th largest c that can be chosen (the lowest index among equals), j < top
 //   weight[t, j] = s[choice] / (sum_j s[choice_j] + 1e-20) * scale
 // With `sigmoid` s is the logistic function of every logit by itself; without `renorm` the weights are s[choice] * scale.
 // The caller sees to it that the kept groups hold at least `top` outputs.
 __global__ __launch_bounds__(kWave) void moe_router_choose_kernel(const float* __restrict__ z, const float* __restrict__ correction,
-                                                                  int E, int n_groups, int keep, int top, float scale, int sigmoid, int renorm,
+                                                                  int E, int n_groups, int keep, int group_best, int top, float scale, int sigmoid, int renorm,
                                                                   int* __restrict__ choice, float* __restrict__ weight) {
     __shared__ float s[kMoeMaxExperts], c[kMoeMaxExperts], gbest[kMoeMaxExperts], picked_s[kMoeMaxExperts];
     __shared__ int picked[kMoeMaxExperts];
@@ -357,9 +366,13 @@ __global__ __launch_bounds__(kWave) void moe_router_choose_kernel(const float* _
     if (n_groups > 1 && keep < n_groups) {
         const int size = E / n_groups;
         for (int g = lane; g < n_groups; g += kWave) {
-            float b = c[g * size];
-            for (int j = 1; j < size; ++j) b = fmaxf(b, c[g * size + j]);
-            gbest[g] = b;
+            float b = c[g * size], b2 = -INFINITY;           // the largest and the second largest
+            for (int j = 1; j < size; ++j) {
+                const float v = c[g * size + j];
+                b2 = fmaxf(b2, fminf(b, v));
+                b = fmaxf(b, v);
+            }
+            gbest[g] = group_best == 2 && size > 1 ? b + b2 : b;
             gopen[g] = 1;
         }
         __syncthreads();
@@ -387,15 +400,16 @@ __global__ __launch_bounds__(kWave) void moe_router_choose_kernel(const float* _
     }
 }
 
-LLOGOS_EXPORT int llogos_moe_router_choose(const float* z, const float* correction, int T, int E, int n_groups, int keep, int top,
+LLOGOS_EXPORT int llogos_moe_router_choose(const float* z, const float* correction, int T, int E, int n_groups, int keep, int group_best, int top,
                                            float scale, int sigmoid, int renorm, int* choice, float* weight, hipStream_t stream) {
     if (T <= 0 || E <= 0 || E > kMoeMaxExperts || top <= 0 || top > E) return LLOGOS_BAD_ARGUMENT;
     if (n_groups > 1 && (E % n_groups || keep < 1 || (long long)min(keep, n_groups) * (E / n_groups) < top)) return LLOGOS_BAD_ARGUMENT;
-    moe_router_choose_kernel<<<T, kWave, 0, stream>>>(z, correction, E, n_groups, keep, top, scale, sigmoid, renorm, choice, weight);
+    if (group_best != 1 && group_best != 2) return LLOGOS_BAD_ARGUMENT;
+    moe_router_choose_kernel<<<T, kWave, 0, stream>>>(z, correction, E, n_groups, keep, group_best, top, scale, sigmoid, renorm, choice, weight);
     return LLOGOS_LAUNCH_CHECK();
 }
 
-// out[t, :] = sum_j weight[t, j] * row_j + (sum of the parts of shared[t, :]), with row_j = y[where[t * top + j], :] when
+// out[t, :] = sum_j weight[t, j] * row_j + shared_scale * (sum of the parts of shared[t, :]), with row_j = y[where[t * top + j], :] when
 // choice[t, j] < n_real and the token's own row a[t, :] otherwise (a router output without matrices returns its input).
 // y float32 [P, W]; a [T, lda] of any storage type; shared float32 [(parts,) T, W] or null.  weight null: every row counts
 // once.  `add`: the result joins what out holds (the float32 stream), and with `rows` the new rows are left in that type too.
@@ -403,7 +417,7 @@ template <typename TA>
 __global__ void moe_combine_weighted_kernel(float* __restrict__ out, const float* __restrict__ y, const int* __restrict__ where,
                                             const int* __restrict__ choice, const float* __restrict__ weight, int top, int n_real,
                                             const TA* __restrict__ a, int lda, const float* __restrict__ shared_rows, int parts,
-                                            size_t part_stride, int T, int W, int add, TA* __restrict__ rows) {
+                                            size_t part_stride, float shared_scale, int T, int W, int add, TA* __restrict__ rows) {
     const int t = blockIdx.x;
     for (int col = blockIdx.y * blockDim.x + threadIdx.x; col < W; col += gridDim.y * blockDim.x) {
         float v = 0.f;
@@ -415,7 +429,7 @@ __global__ void moe_combine_weighted_kernel(float* __restrict__ out, const float
         if (shared_rows) {
             float sh = shared_rows[(size_t)t * W + col];
             for (int q = 1; q < parts; ++q) sh += shared_rows[q * part_stride + (size_t)t * W + col];
-            v += sh;
+            v = fmaf(shared_scale, sh, v);
         }
         if (add) v += out[(size_t)t * W + col];
         if (rows) store_f32(rows + (size_t)t * W + col, v);
@@ -425,16 +439,16 @@ __global__ void moe_combine_weighted_kernel(float* __restrict__ out, const float
 
 LLOGOS_EXPORT int llogos_moe_combine_weighted(float* out, const float* y, const int* where, const int* choice, const float* weight,
                                               int top, int n_real, const void* a, int a_dtype, int lda, const float* shared_rows,
-                                              int parts, long long part_stride, int T, int W, int add, void* rows, hipStream_t stream) {
+                                              int parts, long long part_stride, float shared_scale, int T, int W, int add, void* rows, hipStream_t stream) {
     if (T <= 0 || W <= 0 || top <= 0 || parts < 1 || lda < W || n_real < 0) return LLOGOS_BAD_ARGUMENT;
     const int threads = 256;
     dim3 grid(T, (W + threads - 1) / threads);
     if (a_dtype == DT_F32)
         moe_combine_weighted_kernel<float><<<grid, threads, 0, stream>>>(out, y, where, choice, weight, top, n_real, (const float*)a, lda,
-                                                                         shared_rows, parts, (size_t)part_stride, T, W, add, (float*)rows);
+                                                                         shared_rows, parts, (size_t)part_stride, shared_scale, T, W, add, (float*)rows);
     else if (a_dtype == DT_BF16)
         moe_combine_weighted_kernel<bf16_t><<<grid, threads, 0, stream>>>(out, y, where, choice, weight, top, n_real, (const bf16_t*)a, lda,
-                                                                          shared_rows, parts, (size_t)part_stride, T, W, add, (bf16_t*)rows);
+                                                                          shared_rows, parts, (size_t)part_stride, shared_scale, T, W, add, (bf16_t*)rows);
     else return LLOGOS_BAD_ARGUMENT;
     return LLOGOS_LAUNCH_CHECK();
 }
@@ -488,7 +502,7 @@ template <typename TO>
 __global__ __launch_bounds__(256) void moe_few_kernel(TO* __restrict__ out, const bf16_t* __restrict__ a, const bf16_t* __restrict__ w,
                                                       const int* __restrict__ order, const int* __restrict__ seg, int E, int top,
                                                       int gather, int N, int K, int lda, int act, float scale,
-                                                      const float* __restrict__ row_weight) {
+                                                      const float* __restrict__ row_weight, float limit) {
     __shared__ float red[3][kWave][4];
     __shared__ int s_tile[3];
     if (threadIdx.x == 0) moe_find_tile(seg, E, 16, blockIdx.y, s_tile[0], s_tile[1], s_tile[2]);
@@ -522,13 +536,13 @@ __global__ __launch_bounds__(256) void moe_few_kernel(TO* __restrict__ out, cons
     for (int r = 0; r < 4; ++r) {
         v[r] = ((acc[r] + red[0][lane][r]) + red[1][lane][r]) + red[2][lane][r];
         if (act == 1) { v[r] = fmaxf(v[r], 0.f); v[r] *= v[r]; }
-        if (act != 2) v[r] *= scale;
+        if (act < 2) v[r] *= scale;
     }
     const int n = n0 + 4 * g;
     if (m < m_end && n < N) {
-        if (act == 2) {
+        if (act >= 2) {
             const float rw = row_weight ? row_weight[order[m]] : 1.0f;
-            moe_store2(out + (size_t)m * (N / 2) + n / 2, moe_gated(v[0] * rw, v[1] * rw) * scale, moe_gated(v[2] * rw, v[3] * rw) * scale);
+            moe_store2(out + (size_t)m * (N / 2) + n / 2, moe_gated(v[0] * rw, v[1] * rw, act, limit) * scale, moe_gated(v[2] * rw, v[3] * rw, act, limit) * scale);
         } else moe_store4(out + (size_t)m * N + n, v[0], v[1], v[2], v[3]);
     }
 }
@@ -547,7 +561,7 @@ template <int BM, int BN, typename TO>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3, 3))) void moe_tiles_kernel(
         TO* __restrict__ out, const bf16_t* __restrict__ a, const bf16_t* __restrict__ w, const int* __restrict__ order,
         const int* __restrict__ seg, int E, int top, int gather, int N, int K, int lda, int act, float scale,
-                                                          const float* __restrict__ row_weight) {
+                                                          const float* __restrict__ row_weight, float limit) {
     constexpr int CA = BM * 8 / 256, CW = BN * 8 / 256;           // 16-byte pieces a thread copies a stage
     constexpr int WN = BM == 128 ? BN / 2 : BN / 4, NT = WN / 32, MT = 2;     // a wave's part: 64 rows x WN columns of the tile
     __shared__ __attribute__((aligned(16))) bf16_t As[BM * kMoeBK];
@@ -643,9 +657,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3, 3))) voi
                 for (int r = 0; r < 4; ++r) {
                     v[r] = acc[nt][mt][4 * q + r];
                     if (act == 1) { v[r] = fmaxf(v[r], 0.f); v[r] *= v[r]; }
-                    if (act != 2) v[r] *= scale;
+                    if (act < 2) v[r] *= scale;
                 }
-                if (act == 2) moe_store2(out + (size_t)m * (N / 2) + n / 2, moe_gated(v[0] * rw, v[1] * rw) * scale, moe_gated(v[2] * rw, v[3] * rw) * scale);
+                if (act >= 2) moe_store2(out + (size_t)m * (N / 2) + n / 2, moe_gated(v[0] * rw, v[1] * rw, act, limit) * scale, moe_gated(v[2] * rw, v[3] * rw, act, limit) * scale);
                 else moe_store4(out + (size_t)m * N + n, v[0], v[1], v[2], v[3]);
             }
     }
@@ -654,14 +668,14 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3, 3))) voi
 // form 0: few rows (tiles of 16); 1: tiles of 64 rows; 2: tiles of 128 rows.  -2 for shapes these do not take.
 LLOGOS_EXPORT int llogos_moe_product_bf16(void* out, int out_dtype, const void* a, const void* w, const int* order, const int* seg,
                                           int E, int top, int gather, int P, int N, int K, int lda, int act, float scale,
-                                          const float* row_weight, int form, hipStream_t stream) {
-    if (P <= 0 || N <= 0 || K <= 0 || E <= 0 || top <= 0 || lda < K || act < 0 || act > 2 || form < 0 || form > 2 || (row_weight && act != 2)) return LLOGOS_BAD_ARGUMENT;
+                                          const float* row_weight, float limit, int form, hipStream_t stream) {
+    if (P <= 0 || N <= 0 || K <= 0 || E <= 0 || top <= 0 || lda < K || act < 0 || act > 3 || form < 0 || form > 2 || (row_weight && act < 2) || (act == 3 && !(limit >= 0.f))) return LLOGOS_BAD_ARGUMENT;
     if ((K % 8) || (N % 4) || (lda % 8) || ((uintptr_t)a % 16) || ((uintptr_t)w % 16) || ((uintptr_t)out % 16)) return LLOGOS_UNSUPPORTED;
     if (out_dtype != DT_F32 && out_dtype != DT_BF16) return LLOGOS_BAD_ARGUMENT;
     const int rows = form == 0 ? 16 : (form == 1 ? 64 : 128);
     const int row_tiles = (P + rows - 1) / rows + E;
 #define MOE_GO(KERNEL, NB, TO) KERNEL<<<dim3((N + NB - 1) / NB, row_tiles), 256, 0, stream>>>((TO*)out, (const bf16_t*)a, (const bf16_t*)w, \
-        order, seg, E, top, gather, N, K, lda, act, scale, row_weight)
+        order, seg, E, top, gather, N, K, lda, act, scale, row_weight, limit)
     if (form == 0) { if (out_dtype == DT_F32) MOE_GO(moe_few_kernel<float>, 16, float); else MOE_GO(moe_few_kernel<bf16_t>, 16, bf16_t); }
     else if (form == 1) { if (out_dtype == DT_F32) MOE_GO((moe_tiles_kernel<64, 128, float>), 128, float); else MOE_GO((moe_tiles_kernel<64, 128, bf16_t>), 128, bf16_t); }
     else { if (out_dtype == DT_F32) MOE_GO((moe_tiles_kernel<128, 128, float>), 128, float); else MOE_GO((moe_tiles_kernel<128, 128, bf16_t>), 128, bf16_t); }

@@ -643,8 +643,8 @@ LLOGOS_EXPORT int llogos_sandwich_norm(float* x, const void* a, int a_dtype, int
 //   0 tanh;  1 silu;  2 gelu (tanh form);
 //   3 the piecewise xIELU with a = softplus(p), b = 1/2 + softplus(q):
 //       z > 0: a z^2 + z / 2;   z <= 0: b (exp(z) - 1 - z) + z / 2
-//   4 the square of relu: max(z, 0)^2
-enum { ACT_TANH = 0, ACT_SILU = 1, ACT_GELU_TANH = 2, ACT_XIELU = 3, ACT_RELU2 = 4 };
+//   4 the square of relu: max(z, 0)^2;  5 the sum as it is
+enum { ACT_TANH = 0, ACT_SILU = 1, ACT_GELU_TANH = 2, ACT_XIELU = 3, ACT_RELU2 = 4, ACT_NONE = 5 };
 
 __device__ __forceinline__ float activate(float z, int kind, float a, float b) {
     switch (kind) {
@@ -652,6 +652,7 @@ __device__ __forceinline__ float activate(float z, int kind, float a, float b) {
         case ACT_SILU: return z / (1.0f + expf(-z));
         case ACT_GELU_TANH: return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
         case ACT_RELU2: { const float r = fmaxf(z, 0.f); return r * r; }
+        case ACT_NONE: return z;
         default: return z > 0.f ? fmaf(a * z, z, 0.5f * z) : fmaf(b, expm1f(z) - z, 0.5f * z);
     }
 }
@@ -670,7 +671,7 @@ __global__ void activation_kernel(TO* __restrict__ out, const TI* __restrict__ i
 
 LLOGOS_EXPORT int llogos_activation(void* out, int out_dtype, const void* in, int in_dtype, int parts, long long part_stride,
                                     long long n, int kind, float a, float b, int cols, int ld_in, hipStream_t stream) {
-    if (n <= 0 || parts < 1 || kind < 0 || kind > ACT_RELU2 || cols < 0 || (cols > 0 && ld_in < cols)) return LLOGOS_BAD_ARGUMENT;
+    if (n <= 0 || parts < 1 || kind < 0 || kind > ACT_NONE || cols < 0 || (cols > 0 && ld_in < cols)) return LLOGOS_BAD_ARGUMENT;
     const unsigned blocks = (unsigned)((n + 255) / 256);
 #define ACT(TO, TI) activation_kernel<TO, TI><<<blocks, 256, 0, stream>>>((TO*)out, (const TI*)in, parts, (size_t)part_stride, (size_t)n, kind, a, b, cols, ld_in)
     if (out_dtype == DT_F32 && in_dtype == DT_F32) ACT(float, float);
@@ -679,5 +680,33 @@ LLOGOS_EXPORT int llogos_activation(void* out, int out_dtype, const void* in, in
     else if (out_dtype == DT_F32 && in_dtype == DT_BF16) ACT(float, bf16_t);
     else return LLOGOS_BAD_ARGUMENT;
 #undef ACT
+    return LLOGOS_LAUNCH_CHECK();
+}
+
+// Both halves of a product's rows [gate (N) | up (N)] (maybe in parts) bounded and joined: with g = min(gate, limit) and
+// u = up kept within -limit .. limit, out = g * sigmoid(1.702 g) * (u + 1).
+template <typename TO, typename TI>
+__global__ void clamped_glu_kernel(TO* __restrict__ out, const TI* __restrict__ in, int parts, size_t part_stride, size_t n, int N, float limit) {
+    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= n) return;
+    const size_t at = (i / N) * (size_t)(2 * N) + i % N;
+    float g = load_f32(in + at), u = load_f32(in + at + N);
+    for (int q = 1; q < parts; ++q) { g += load_f32(in + q * part_stride + at); u += load_f32(in + q * part_stride + at + N); }
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    store_f32(out + i, g / (1.0f + expf(-1.702f * g)) * (u + 1.0f));
+}
+
+LLOGOS_EXPORT int llogos_clamped_glu(void* out, int out_dtype, const void* in, int in_dtype, int parts, long long part_stride, int T, int N,
+                                     float limit, hipStream_t stream) {
+    if (T <= 0 || N <= 0 || parts < 1 || !(limit >= 0.f)) return LLOGOS_BAD_ARGUMENT;
+    const size_t n = (size_t)T * N;
+    const unsigned blocks = (unsigned)((n + 255) / 256);
+#define CG(TO, TI) clamped_glu_kernel<TO, TI><<<blocks, 256, 0, stream>>>((TO*)out, (const TI*)in, parts, (size_t)part_stride, n, N, limit)
+    if (out_dtype == DT_F32 && in_dtype == DT_F32) CG(float, float);
+    else if (out_dtype == DT_BF16 && in_dtype == DT_F32) CG(bf16_t, float);
+    else if (out_dtype == DT_BF16 && in_dtype == DT_BF16) CG(bf16_t, bf16_t);
+    else return LLOGOS_BAD_ARGUMENT;
+#undef CG
     return LLOGOS_LAUNCH_CHECK();
 }

@@ -433,7 +433,7 @@ def argmax(logits: torch.Tensor) -> torch.Tensor:
 # parts with a fixed-size state per sequence
 # ----------------------------------------------------------------------------
 MAX_CONV_TAPS = 16
-ACTIVATIONS = {"tanh": 0, "silu": 1, "gelu_tanh": 2, "xielu": 3, "relu2": 4}
+ACTIVATIONS = {"tanh": 0, "silu": 1, "gelu_tanh": 2, "xielu": 3, "relu2": 4, "none": 5}
 
 
 def causal_conv(ctx, h: torch.Tensor, w: torch.Tensor, state: torch.Tensor, out_dtype: torch.dtype,
@@ -586,18 +586,20 @@ def sandwich_norm(x: torch.Tensor, a: torch.Tensor, post_w: torch.Tensor, next_w
 
 
 def activation(x: torch.Tensor, kind: str, out_dtype: torch.dtype, a: float = 0.0, b: float = 0.0,
-               cols: Optional[int] = None) -> torch.Tensor:
+               cols: Optional[int] = None, first: int = 0) -> torch.Tensor:
     """act(x) element by element; x [T, N] or float32 partial sums [parts, T, N] that are added first.
     kinds: tanh, silu, gelu_tanh, xielu (z > 0: a z^2 + z / 2; z <= 0: b (exp(z) - 1 - z) + z / 2), relu2
-    (the square of max(z, 0)).  cols: only the first `cols` values of every row are taken (the result is
-    [T, cols]): a product whose rows hold something else behind them."""
+    (the square of max(z, 0)), none (the sums as they are).  cols: only `cols` values of every row are taken, from
+    column `first` on (the result is [T, cols]): a product whose rows hold something else around them."""
     _dev(x)
     _need(kind in ACTIVATIONS, f"activation: unknown kind '{kind}'; known: {sorted(ACTIVATIONS)}")
     parts, part_stride = _parts(x)
     _need(parts == 1 or x.dtype == torch.float32, "activation: parts must be float32")
     T, N = x.shape[-2:]
-    C = N if cols is None else int(cols)
-    _need(0 < C <= N, "activation: cols outside 1..N")
+    C = N - first if cols is None else int(cols)
+    _need(first >= 0 and 0 < C <= N - first, "activation: columns outside the rows")
+    if first:
+        x = x[..., first:]                   # (the kernel is told where the rows lie)
     out = torch.empty((T, C), dtype=out_dtype, device=x.device)
     if out.numel():
         _check(_lib().llogos_activation(_p(out), _DT[out_dtype], _p(x), _dt(x), parts, ctypes.c_longlong(part_stride),
@@ -631,11 +633,11 @@ def moe_route(ids: Optional[torch.Tensor], table: torch.Tensor, n_experts: int):
 
 
 def moe_router(h: torch.Tensor, router_w: torch.Tensor, correction: Optional[torch.Tensor], n_groups: int, keep: int, top: int,
-               scale: float, scores: str = "softmax", renorm: bool = True):
+               scale: float, scores: str = "softmax", renorm: bool = True, group_score: str = "best"):
     """A router's choice for every row of h [T, K] (any storage type): logits z = h . router_w^T in 32-bit
     (router_w float32 [E, K]), s = softmax(z) over all E outputs, the choice's scores s + correction (float32 [E]
     or None), of which only those in the `keep` best of n_groups equal groups of neighbouring outputs (a group's
-    score is its largest) can be chosen; the `top` largest are chosen (the lowest index among equals).
+    score is its largest, with group_score "best_two" the sum of its two largest) can be chosen; the `top` largest are chosen (the lowest index among equals).
     Returns (choice int32 [T, top], weight float32 [T, top]) with weight = s[choice] / (their sum + 1e-20) * scale.
     scores "sigmoid": s is the logistic function of every logit by itself; renorm False: weight = s[choice] * scale."""
     _dev(router_w, correction)
@@ -646,6 +648,7 @@ def moe_router(h: torch.Tensor, router_w: torch.Tensor, correction: Optional[tor
     _need(0 < top <= E <= MOE_MAX_EXPERTS, f"moe_router: top within 1..E, at most {MOE_MAX_EXPERTS} outputs")
     _need(correction is None or (correction.dtype == torch.float32 and correction.shape == (E,)), "moe_router: correction must be float32 [E]")
     _need(scores in ("softmax", "sigmoid"), "moe_router: scores 'softmax' or 'sigmoid'")
+    _need(group_score in ("best", "best_two"), "moe_router: group_score 'best' or 'best_two'")
     n_groups, keep = max(1, int(n_groups)), int(keep)
     if n_groups > 1:
         _need(E % n_groups == 0 and keep >= 1 and min(keep, n_groups) * (E // n_groups) >= top,
@@ -655,15 +658,15 @@ def moe_router(h: torch.Tensor, router_w: torch.Tensor, correction: Optional[tor
                                            T, E, Kk, _stream()), "moe_router_logits")
     choice = torch.empty((T, top), dtype=torch.int32, device=h.device)
     weight = torch.empty((T, top), dtype=torch.float32, device=h.device)
-    _check(_lib().llogos_moe_router_choose(_p(z), _p(correction), T, E, n_groups, keep, top, ctypes.c_float(scale),
+    _check(_lib().llogos_moe_router_choose(_p(z), _p(correction), T, E, n_groups, keep, 2 if group_score == "best_two" else 1, top, ctypes.c_float(scale),
                                            int(scores == "sigmoid"), int(bool(renorm)), _p(choice), _p(weight), _stream()), "moe_router_choose")
     return choice, weight
 
 
 def moe_combine_weighted(y: torch.Tensor, where: torch.Tensor, choice: torch.Tensor, weight: Optional[torch.Tensor], n_real: int,
                          h: torch.Tensor, shared: Optional[torch.Tensor] = None, stream: Optional[torch.Tensor] = None,
-                         rows: bool = False):
-    """float32 [T, W]: sum_j weight[t, j] * row_j + shared[t], where row_j is the pair's row y[where[t * top + j]]
+                         rows: bool = False, shared_scale: float = 1.0):
+    """float32 [T, W]: sum_j weight[t, j] * row_j + shared_scale * shared[t], where row_j is the pair's row y[where[t * top + j]]
     when choice[t, j] < n_real and the token's own row h[t] otherwise (a router output that has no matrices and
     returns its input).  y float32 [T * top, W]; h [T, W] of any storage type; shared float32 [T, W] or parts.
     weight None: every row counts once.  stream: the result joins this float32 [T, W] in place, and what comes back is
@@ -687,19 +690,20 @@ def moe_combine_weighted(y: torch.Tensor, where: torch.Tensor, choice: torch.Ten
     new_rows = torch.empty((T, W), dtype=h.dtype, device=y.device) if rows else None
     _check(_lib().llogos_moe_combine_weighted(_p(out), _p(y), _p(where), _p(choice), _p(weight), top, int(n_real), _p(h), _dt(h),
                                               h.stride(0) if T > 1 else max(W, h.stride(0)), _p(shared), parts,
-                                              ctypes.c_longlong(part_stride), T, W, 0 if stream is None else 1, _p(new_rows), _stream()),
-           "moe_combine_weighted")
+                                              ctypes.c_longlong(part_stride), ctypes.c_float(shared_scale), T, W, 0 if stream is None else 1,
+                                              _p(new_rows), _stream()), "moe_combine_weighted")
     return out if stream is None else new_rows
 
 
 def moe_product(a: torch.Tensor, w: torch.Tensor, order: torch.Tensor, seg: torch.Tensor, top: int, gather: bool,
                 out_dtype: torch.dtype, relu2: bool = False, scale: float = 1.0, gated: bool = False,
-                pair_weight: Optional[torch.Tensor] = None) -> torch.Tensor:
+                pair_weight: Optional[torch.Tensor] = None, limit: Optional[float] = None) -> torch.Tensor:
     """[P, N]: sorted row r, which belongs to the expert e whose segment holds it, is a_row(r) . w[e]^T, with
     a_row(r) = a[order[r] // top] (gather: a holds the step's token rows) or a[r] (a is sorted already);
     w [E, N, K]; relu2 squares max(., 0) in the epilogue, scale multiplies the result.  gated: the rows of
     w[e] are gate and up rows in turn (gate 0, up 0, gate 1, ...) and the result is [P, N / 2], column i
-    silu(gate_i sum) * (up_i sum); pair_weight float32 [P] (with gated): pair p's row counts as pair_weight[p] times
+    silu(gate_i sum) * (up_i sum), with `limit` g * sigmoid(1.702 g) * (u + 1) of the sums bounded to g = min(gate_i, limit) and
+    u = up_i within -limit .. limit; pair_weight float32 [P] (with gated): pair p's row counts as pair_weight[p] times
     itself, which multiplies both sums.  `seg` may hold more segments than w has experts: rows in those belong
     to choices without a matrix and are left unwritten."""
     _dev(a, w, order, seg)
@@ -715,7 +719,9 @@ def moe_product(a: torch.Tensor, w: torch.Tensor, order: torch.Tensor, seg: torc
     if pair_weight is not None:
         _dev(pair_weight)
         _need(gated and pair_weight.dtype == torch.float32 and pair_weight.numel() == P, "moe_product: pair_weight float32 [P], with the gated epilogue")
-    act = 2 if gated else (1 if relu2 else 0)
+    _need(limit is None or (gated and limit >= 0.0), "moe_product: a limit goes with the gated epilogue")
+    act = (2 if limit is None else 3) if gated else (1 if relu2 else 0)
+    lim = ctypes.c_float(limit or 0.0)
     out = torch.empty((P, N // 2 if gated else N), dtype=out_dtype, device=a.device)
     if a.dtype == torch.bfloat16 and MOE_PRODUCT != "plain" and a.stride(1) == 1:
         # on the matrix cores: tiles of 16 sorted rows straight from memory for steps of few rows, tiles of 64 or
@@ -724,12 +730,12 @@ def moe_product(a: torch.Tensor, w: torch.Tensor, order: torch.Tensor, seg: torc
         if MOE_PRODUCT in ("few", "tiles64", "tiles128"):
             form = ("few", "tiles64", "tiles128").index(MOE_PRODUCT)
         code = _lib().llogos_moe_product_bf16(_p(out), _DT[out_dtype], _p(a), _p(w), _p(order), _p(seg), E, top, 1 if gather else 0,
-                                              P, N, Kk, a.stride(0), act, ctypes.c_float(scale), _p(pair_weight), form, _stream())
+                                              P, N, Kk, a.stride(0), act, ctypes.c_float(scale), _p(pair_weight), lim, form, _stream())
         if code != -2:
             _check(code, "moe_product")
             return out
     _check(_lib().llogos_moe_product(_p(out), _DT[out_dtype], _p(a), _dt(a), _p(w), _dt(w), _p(order), _p(seg), E, top,
-                                     1 if gather else 0, P, N, Kk, a.stride(0), act, ctypes.c_float(scale), _p(pair_weight), _stream()),
+                                     1 if gather else 0, P, N, Kk, a.stride(0), act, ctypes.c_float(scale), _p(pair_weight), lim, _stream()),
            "moe_product")
     return out
 
@@ -1180,6 +1186,187 @@ def gated_row_norm(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, ep
         _check(_lib().llogos_gated_row_norm(_p(y), _DT[out_dtype], _p(o), _p(weight), _p(gate), gate.stride(-2) if T > 1 else max(N, gate.stride(-2)),
                                             parts, ctypes.c_longlong(part_stride), ctypes.c_float(eps), T, N, _stream()), "gated_row_norm")
     return y
+
+
+DELTA_CHUNK = 32             # tokens a chunk of the recurrence (kDeltaChunk in csrc/delta_recurrence.hip)
+DELTA_MAX_DIM = 256          # key channels a head
+DELTA_MAX_V = 1024           # value channels a head
+
+
+def delta_shape_ok(dim: int, v_dim: int) -> bool:
+    """Whether the kernels of the gated delta rule take heads of `dim` key and `v_dim` value channels."""
+    return 0 < dim <= DELTA_MAX_DIM and 0 < v_dim <= DELTA_MAX_V
+
+
+def delta_step_threads(dim: int, v_dim: int) -> int:
+    """Threads a block of the kernel for single-token steps (a thread holds up to 64 values of the state); 0: a head too
+    large for it, whose single tokens go through the kernels for longer steps."""
+    return _lib().llogos_delta_step_threads(dim, v_dim)
+
+
+@dataclass
+class DeltaShape:
+    """What the kernels of the gated delta rule are told about a mixer: heads, key heads, key and value channels a head, taps
+    of the convolution; `channelwise`: a decay a key channel instead of one a head; `b_col`: where beta's logits (one a
+    head) lie in the projected rows, whose first columns are q (G D), k (G D) and v (H V)."""
+    H: int
+    G: int
+    D: int
+    V: int
+    taps: int
+    channelwise: bool
+    b_col: int
+
+    @property
+    def width(self) -> int:
+        return 2 * self.G * self.D + self.H * self.V
+
+    @property
+    def n_decay(self) -> int:
+        return self.H * self.D if self.channelwise else self.H
+
+    @property
+    def state_floats(self) -> int:
+        """A slot's state row: S of every head [H][D][V], then the last `taps` projected rows, position p in row p % taps."""
+        return self.H * self.D * self.V + self.taps * self.width
+
+
+def _f32_rows(t: torch.Tensor, rows: int, cols: int, who: str) -> Tuple[int, int, int]:
+    """(row stride, parts, part stride) of float32 rows [rows, >= cols] or partial sums [parts, rows, >= cols] of them (views of
+    some columns of wider rows will do)."""
+    _need(t.is_cuda and t.dtype == torch.float32 and t.dim() in (2, 3) and t.stride(-1) == 1, f"{who}: float32 rows on the GPU")
+    _need(t.shape[-2] == rows and t.shape[-1] >= cols, f"{who}: {rows} rows of at least {cols} values")
+    parts, part_stride = _parts(t)
+    return (t.stride(-2) if rows > 1 else max(cols, t.stride(-2))), parts, part_stride
+
+
+def _delta_args(ctx, sh: DeltaShape, rows, conv, z, dt_bias, a_log, state, who: str):
+    _dev(conv, dt_bias, a_log, state, ctx.slots, ctx.tok_seq, ctx.tok_pos, ctx.cu_dev)
+    _need(sh.H > 0 and sh.G > 0 and sh.H % sh.G == 0 and delta_shape_ok(sh.D, sh.V) and 1 <= sh.taps <= MAX_CONV_TAPS, f"{who}: head shape")
+    _need(conv.dtype == torch.float32 and tuple(conv.shape) == (sh.taps, sh.width), f"{who}: taps float32 [taps, width]")
+    for t, n, name in ((dt_bias, sh.n_decay, "dt_bias"), (a_log, sh.H, "A_log")):
+        _need(t.dtype == torch.float32 and t.numel() == n, f"{who}: {name} float32 [{n}]")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.shape[1] == sh.state_floats, f"{who}: state must be float32 [slots, {sh.state_floats}]")
+    r = _f32_rows(rows, ctx.n_tokens, max(sh.width, sh.b_col + sh.H), who + " rows")
+    d = _f32_rows(z, ctx.n_tokens, sh.n_decay, who + " decay")
+    return r, d
+
+
+def _delta_offsets(ctx) -> torch.Tensor:
+    """Token offsets of the step's sequences on the device (made here for a captured step, which has none)."""
+    if ctx.cu_dev is not None:
+        return ctx.cu_dev
+    _need(ctx.n_tokens == ctx.batch, "a step of several tokens a sequence needs the token offsets")
+    cu = ctx.shared.get("offsets")
+    if cu is None:
+        cu = ctx.shared["offsets"] = torch.arange(ctx.batch + 1, dtype=torch.int32, device=ctx.slots.device)
+    return cu
+
+
+def delta_step(ctx, sh: DeltaShape, rows: torch.Tensor, conv: torch.Tensor, z: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor,
+               gate: torch.Tensor, gate_silu: bool, norm_w: torch.Tensor, eps: float, state: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """A single-token step of the gated delta rule from its projected rows to the rows of its output product [T, H V]:
+    convolution, silu, unit vectors, decay exp(-exp(a_log) softplus(z + dt_bias)), beta, the state's update and
+    read-out, the norm over a head with weight norm_w [V], times silu(gate) or sigmoid(gate)."""
+    (ld, parts, ps), (ldz, zp, zps) = _delta_args(ctx, sh, rows, conv, z, dt_bias, a_log, state, "delta_step")
+    _need(ctx.n_tokens == ctx.batch, "delta_step: one token a sequence")
+    ldg, gp, gps = _f32_rows(gate, ctx.n_tokens, sh.H * sh.V, "delta_step gate")
+    _dev(norm_w)
+    _need(norm_w.dtype == torch.float32 and norm_w.shape == (sh.V,), "delta_step: norm weight float32 [V]")
+    y = torch.empty((ctx.n_tokens, sh.H * sh.V), dtype=out_dtype, device=rows.device)
+    _check(_lib().llogos_delta_step(_p(y), _DT[out_dtype], _p(rows), ld, parts, ctypes.c_longlong(ps), _p(conv), sh.taps, _p(state),
+                                    ctypes.c_longlong(state.stride(0)), _p(ctx.slots), _p(ctx.tok_pos), ctx.batch, sh.H, sh.G, sh.D, sh.V, _p(z),
+                                    ldz, zp, ctypes.c_longlong(zps), _p(dt_bias), _p(a_log), int(sh.channelwise), sh.b_col, _p(gate), ldg, gp,
+                                    ctypes.c_longlong(gps), int(bool(gate_silu)), _p(norm_w), ctypes.c_float(eps), _stream()), "delta_step")
+    return y
+
+
+def delta_prepare(ctx, sh: DeltaShape, rows: torch.Tensor, conv: torch.Tensor, z: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor,
+                  state: torch.Tensor):
+    """(act [T, width], logd [T, H or H D], beta [T, H]), float32: what delta_scan reads of a step of any length (q, k, v behind
+    convolution, silu and the unit norms; log2 of the decays; sigmoids).  The convolution's part of the state is brought up to date."""
+    (ld, parts, ps), (ldz, zp, zps) = _delta_args(ctx, sh, rows, conv, z, dt_bias, a_log, state, "delta_prepare")
+    cu = _delta_offsets(ctx)
+    T, dev = ctx.n_tokens, rows.device
+    act = torch.empty((T, sh.width), dtype=torch.float32, device=dev)
+    logd = torch.empty((T, sh.n_decay), dtype=torch.float32, device=dev)
+    beta = torch.empty((T, sh.H), dtype=torch.float32, device=dev)
+    _check(_lib().llogos_delta_prepare(_p(act), _p(logd), _p(beta), _p(rows), ld, parts, ctypes.c_longlong(ps), _p(conv), sh.taps, _p(state),
+                                       ctypes.c_longlong(state.stride(0)), _p(ctx.slots), _p(ctx.tok_seq), _p(ctx.tok_pos), _p(cu), T,
+                                       ctx.batch, sh.H, sh.G, sh.D, sh.V, _p(z), ldz, zp, ctypes.c_longlong(zps), _p(dt_bias), _p(a_log),
+                                       int(sh.channelwise), sh.b_col, _stream()), "delta_prepare")
+    return act, logd, beta
+
+
+def delta_scan(ctx, sh: DeltaShape, act: torch.Tensor, logd: torch.Tensor, beta: torch.Tensor, state: torch.Tensor) -> torch.Tensor:
+    """o float32 [T, H V] of the recurrence over the step's rows of each sequence in turn, from what delta_prepare left; S of
+    every head (the front of each slot's state row) is read and brought up to date."""
+    _dev(act, logd, beta, state, ctx.slots, ctx.cu_dev)
+    T = ctx.n_tokens
+    for t, n, name in ((act, sh.width, "act"), (logd, sh.n_decay, "logd"), (beta, sh.H, "beta")):
+        _need(t.dtype == torch.float32 and tuple(t.shape) == (T, n), f"delta_scan: {name} must be float32 [{T}, {n}]")
+    cu = _delta_offsets(ctx)
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.shape[1] == sh.state_floats and delta_shape_ok(sh.D, sh.V), "delta_scan: state")
+    chunks = ctx.batch if ctx.is_decode else sum(-(-(ctx.cu_seqlens[i + 1] - ctx.cu_seqlens[i]) // DELTA_CHUNK) for i in range(ctx.batch))
+    floats = _lib().llogos_delta_workspace(chunks, sh.H, sh.D, sh.V)
+    ws = torch.empty(floats, dtype=torch.float32, device=act.device)
+    o = torch.empty((T, sh.H * sh.V), dtype=torch.float32, device=act.device)
+    _check(_lib().llogos_delta_scan(_p(o), _p(act), _p(logd), _p(beta), _p(ws), ctypes.c_longlong(floats), _p(state), ctypes.c_longlong(state.stride(0)),
+                                    _p(ctx.slots), _p(cu), ctx.batch, chunks, sh.H, sh.G, sh.D, sh.V, int(sh.channelwise), _stream()), "delta_scan")
+    return o
+
+
+def delta_out(o: torch.Tensor, gate: torch.Tensor, gate_silu: bool, weight: torch.Tensor, eps: float, n_heads: int,
+              out_dtype: torch.dtype) -> torch.Tensor:
+    """o / sqrt(mean(o^2) + eps) * weight over every head's channels (weight [V], shared by the heads), times silu(gate) or
+    sigmoid(gate): float32 o [T, H V]; gate float32 logits [T, H V] (maybe columns of wider rows) or partial sums of them."""
+    _dev(o, weight)
+    _need(o.dtype == torch.float32 and o.dim() == 2 and n_heads > 0 and o.shape[1] % n_heads == 0, "delta_out: o must be float32 [T, heads * V]")
+    T, V = o.shape[0], o.shape[1] // n_heads
+    _need(weight.dtype == torch.float32 and weight.shape == (V,), "delta_out: weight float32 [V]")
+    ldg, gp, gps = _f32_rows(gate, T, n_heads * V, "delta_out gate")
+    y = torch.empty((T, n_heads * V), dtype=out_dtype, device=o.device)
+    if T:
+        _check(_lib().llogos_delta_out(_p(y), _DT[out_dtype], _p(o), _p(gate), ldg, gp, ctypes.c_longlong(gps), int(bool(gate_silu)), _p(weight),
+                                       ctypes.c_float(eps), T, n_heads, V, _stream()), "delta_out")
+    return y
+
+
+def clamped_glu(gu: torch.Tensor, limit: float, out_dtype: torch.dtype) -> torch.Tensor:
+    """g * sigmoid(1.702 g) * (u + 1) with g = min(gate, limit) and u = up within -limit .. limit, from rows [gate | up]
+    ([T, 2 N] or float32 partial sums [parts, T, 2 N])."""
+    _dev(gu)
+    parts, part_stride = _parts(gu)
+    _need(gu.shape[-1] % 2 == 0 and limit >= 0.0, "clamped_glu: rows must be [gate | up], the limit not negative")
+    _need(gu.dtype == torch.float32 or (parts == 1 and gu.dtype == out_dtype), "clamped_glu: float32 rows or the output's type")
+    T, N = gu.shape[-2], gu.shape[-1] // 2
+    out = torch.empty((T, N), dtype=out_dtype, device=gu.device)
+    if T:
+        _check(_lib().llogos_clamped_glu(_p(out), _DT[out_dtype], _p(gu), _dt(gu), parts, ctypes.c_longlong(part_stride), T, N,
+                                         ctypes.c_float(limit), _stream()), "clamped_glu")
+    return out
+
+
+def pair_norm(a: torch.Tensor, b: torch.Tensor, wa: torch.Tensor, wb: torch.Tensor, eps: float, x: Optional[torch.Tensor] = None,
+              next_w: Optional[torch.Tensor] = None, next_eps: float = 0.0, out_dtype: torch.dtype = torch.float32) -> Optional[torch.Tensor]:
+    """v = rmsnorm(a) * wa + rmsnorm(b) * wb for two products [T, H] (each maybe in float32 parts [parts, T, H]).  Without x: v,
+    float32.  With the float32 stream x: x += v in place, and with next_w the rows rmsnorm(x) * next_w in `out_dtype` come back."""
+    _dev(a, b, wa, wb, x, next_w)
+    T, H = a.shape[-2:]
+    _need(tuple(b.shape[-2:]) == (T, H) and H <= 16384, "pair_norm: two products of one shape, rows of at most 16,384 values")
+    (ap, aps), (bp, bps) = _parts(a), _parts(b)
+    _need((ap == 1 or a.dtype == torch.float32) and (bp == 1 or b.dtype == torch.float32), "pair_norm: parts must be float32")
+    for w in (wa, wb, next_w):
+        _need(w is None or (w.dtype == torch.float32 and w.shape == (H,)), "pair_norm: weights must be float32 [H]")
+    _need(x is None or (x.dtype == torch.float32 and tuple(x.shape) == (T, H)), "pair_norm: x must be float32 [T, H]")
+    _need(next_w is None or x is not None, "pair_norm: the next norm reads the stream")
+    delta = torch.empty((T, H), dtype=torch.float32, device=a.device) if x is None else None
+    h = torch.empty((T, H), dtype=out_dtype, device=a.device) if next_w is not None else None
+    if T:
+        _check(_lib().llogos_pair_norm(_p(x), _p(a), _dt(a), ap, ctypes.c_longlong(aps), _p(b), _dt(b), bp, ctypes.c_longlong(bps), _p(wa), _p(wb),
+                                       ctypes.c_float(eps), _p(next_w), ctypes.c_float(next_eps), _p(h), _DT[out_dtype], _p(delta), T, H, _stream()),
+               "pair_norm")
+    return delta if x is None else h
 
 
 def stream_add(x: torch.Tensor, delta: Optional[torch.Tensor] = None, again: Optional[torch.Tensor] = None,
@@ -2095,7 +2282,7 @@ def capped_attention(ctx, q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
             if head_sink is not None:
                 _dev(head_sink)
                 _need(head_sink.dtype == torch.float32 and head_sink.shape == (n_heads,), "attention: head_sink must be float32 [n_heads]")
-            if ctx.is_decode and window > 0:
+            if ctx.is_decode and window > 0 and softcap > 0.0:
                 code = -2
             elif ctx.is_decode:
                 width = table.shape[1]
@@ -2103,7 +2290,7 @@ def capped_attention(ctx, q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
                 ws = _attn_workspace(q.device, lib.llogos_capped_attn_decode_workspace(T, n_heads, n_kv_heads, v_dim, width))
                 code = lib.llogos_capped_attn_decode_bf16(
                     _p(out), _p(q), q.stride(0), _p(k_pool), _p(v_pool), _p(table), table.stride(0), width, _p(ctx.tok_pos), T,
-                    n_heads, n_kv_heads, head_dim, v_dim, ctypes.c_float(scale), ctypes.c_float(softcap), _p(head_sink), _p(gate),
+                    n_heads, n_kv_heads, head_dim, v_dim, ctypes.c_float(scale), ctypes.c_float(softcap), int(window), _p(head_sink), _p(gate),
                     gate_stride, _p(ws), ctypes.c_longlong(ws.numel()), _stream())
             else:
                 cu = ctx.cu_dev

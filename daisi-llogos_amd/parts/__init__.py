@@ -9,12 +9,14 @@ from .attention import Attention
 from .conv import CausalConv
 from .wkv import WKV
 from .latent_attention import LatentAttention
-from .mlp import ActivatedMLP, SwiGLU
+from .mlp import ActivatedMLP, ClampedGLU, SwiGLU
 from .capped_attention import CappedAttention
 from .moe import RoutedMoE, TableMoE
 from .loop import LoopAdd, LoopEntry
 from .token_side import TokenSide
 from .lightning import Lightning
+from .delta import Delta
+from .side_by_side import SideBySide
 from .rglru import RGLRU
 from .diff_attention import DiffAttention
 from .block import OutputNormBlock, ParallelBlock, PostNormBlock, PreNormBlock, SandwichBlock

@@ -29,10 +29,10 @@ class Attention(Mixer):
                  position: Rotary, bias: bool = False, qk_norm: bool = False, eps: float = 1e-6,
                  window: int = 0, sinks: int = 0, scale: Optional[float] = None,
                  v_dim: Optional[int] = None, unit_qk: bool = False,
-                 names: Sequence[str] = ("q_proj", "k_proj", "v_proj", "o_proj"), suffix: str = ".weight"):
+                 names: Sequence[str] = ("q_proj", "k_proj", "v_proj", "o_proj"), suffix: str = ".weight", bias_suffix: str = ".bias"):
         """v_dim: width of a head's values when it is not head_dim.  unit_qk: after the rotation every head's
         query and key are divided by their root mean square (eps inside the root, no weight).  names, suffix:
-        the four matrices' tensor names behind `prefix`.  With either of the first two the step goes through
+        the four matrices' tensor names behind `prefix` (bias_suffix: what the biases' names have there).  With either of the first two the step goes through
         the preparation kernel for any head shape (ops.kernels.rotary_prepare) instead of the dense decoder's."""
         if n_heads % n_kv_heads:
             raise ValueError(f"{n_heads} heads are not a multiple of {n_kv_heads} kv heads")
@@ -42,8 +42,8 @@ class Attention(Mixer):
         if self.general:
             if max(head_dim, self.v_dim) > K.GENERIC_MAX_HEAD_DIM:
                 raise ValueError(f"heads of {head_dim} and {self.v_dim} dimensions are wider than the attention kernels take")
-            if bias or qk_norm:
-                raise ValueError("biases and the norm before the rotation are not built beside unit-length queries or values of their own width")
+            if qk_norm:
+                raise ValueError("the norm before the rotation is not built beside unit-length queries or values of their own width")
         elif head_dim % 16 or head_dim > K.MAX_HEAD_DIM:
             raise ValueError(f"head_dim {head_dim} must be a multiple of 16, at most {K.MAX_HEAD_DIM}")
         self.prefix = prefix
@@ -55,7 +55,8 @@ class Attention(Mixer):
         self.window, self.sinks = int(window), int(sinks)
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(head_dim)
         q_w, kv_w = n_heads * head_dim, n_kv_heads * head_dim
-        self.qkv = Linear([prefix + n for n in names[:3]], hidden, [q_w, kv_w, n_kv_heads * self.v_dim], bias=bias, suffix=suffix)
+        self.qkv = Linear([prefix + n for n in names[:3]], hidden, [q_w, kv_w, n_kv_heads * self.v_dim], bias=bias, suffix=suffix,
+                          bias_suffix=bias_suffix)
         self.o = Linear([prefix + names[3]], n_heads * self.v_dim, [hidden], suffix=suffix)
         self.q_norm_w: Optional[torch.Tensor] = None
         self.k_norm_w: Optional[torch.Tensor] = None
@@ -125,13 +126,16 @@ class Attention(Mixer):
         rows = self.qkv.product(h, f32_ok=True) if cache.writes else self.qkv.product(h, rows_out=nh * hd, f32_ok=True)
         mark(ctx, "qkv")
         rot, pairing = (self.position.rot, self.position.pairing) if self.position is not None else (0, 0)
-        q = K.rotary_prepare(ctx, rows, None, self.rt.dtype, nh, nkv, hd, vd, 1, rot, pairing, cs,
+        q = K.rotary_prepare(ctx, rows, self.qkv.bias_rows(None if cache.writes else nh * hd), self.rt.dtype, nh, nkv, hd, vd, 1, rot, pairing, cs,
                              None, None, self.unit_qk, self.eps, cache.k_pool, cache.v_pool, cache.table, writes=cache.writes)
         mark(ctx, "rotation")
         spec = self.kv_spec()
         if vd == hd and spec.head_dim == hd:
             a = K.attention(ctx, q, q.stride(0), cache.k_pool, cache.v_pool, cache.table, nh, nkv, hd, self.scale,
                             self.window, self.sinks)
+        elif self.sinks == 0 and self.scale > 0.0:
+            # (keys and values of different widths: the matrix cores for the head shapes they take, else any shape's kernel)
+            a = K.capped_attention(ctx, q, cache.k_pool, cache.v_pool, cache.table, nh, nkv, hd, vd, self.scale, window=self.window)
         else:
             a = K.attention_generic(q, q.stride(0), cache.k_pool, cache.v_pool, cache.table, ctx.tok_seq, ctx.tok_pos,
                                     nh, nkv, hd, self.scale, self.window, self.sinks, v_dim=vd)

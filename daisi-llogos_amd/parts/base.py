@@ -205,6 +205,17 @@ class Mixer(Part):
     # first product); a block whose producer can write either type asks it for that one
     takes_float32_rows = False
 
+    # True: forward takes a list of LayerCaches, one for each of cache_parts() (a mixer put together from others)
+    takes_caches = False
+
+    def cache_parts(self) -> List[Part]:
+        """The parts of this mixer that keep something for each sequence: itself, or the mixers it is made of."""
+        return [self]
+
+    def caches_of(self, caches: List[LayerCache]):
+        """What forward takes of its cache_parts()' LayerCaches."""
+        return list(caches) if self.takes_caches else caches[0]
+
     def kv_spec(self) -> Optional[KVSpec]:
         return None
 
@@ -295,7 +306,7 @@ class Block(Part):
         """The parts that keep something in the cache for each sequence, in the order in which
         forward() takes their LayerCaches: the mixers, unless a block has other parts with state
         (each such part has kv_spec() and state_spec() like a mixer)."""
-        return self.mixers()
+        return [p for m in self.mixers() for p in m.cache_parts()]
 
     def parts(self) -> List[Part]:
         raise NotImplementedError

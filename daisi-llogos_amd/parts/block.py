@@ -53,7 +53,7 @@ class PreNormBlock(Block):
         return norm.forward(x, delta, lazy=True) if lazy and norm.takes_row_squares else norm.forward(x, delta)
 
     def forward(self, ctx: StepContext, x: torch.Tensor, pending, caches, next_norm: Optional[Norm] = None):
-        cache = caches[0] if isinstance(caches, (list, tuple)) else caches
+        cache = self.mixer.caches_of(caches) if isinstance(caches, (list, tuple)) else caches
         # A part that says so may add its output to x itself and leave the next norm's rows half made
         # (then `a` or `d` is what it left, and the norm that takes it needs no kernel of its own).
         last = self.tail if self.tail is not None else next_norm            # who reads the stream behind the sublayers
@@ -102,7 +102,8 @@ class SandwichBlock(Block):
         return [self.ffn] if self.ffn is not None else []
 
     def cache_parts(self) -> List[Part]:
-        return [p for p in (self.mixer_conv, self.mixer, self.ffn_conv) if p is not None]
+        conv = lambda p: [p] if p is not None else []
+        return conv(self.mixer_conv) + self.mixer.cache_parts() + conv(self.ffn_conv)
 
     def parts(self) -> List[Part]:
         return [p for p in (self.mixer_norm, self.mixer_conv, self.mixer, self.post_mixer_norm, self.ffn_norm, self.ffn_conv,
@@ -132,7 +133,7 @@ class SandwichBlock(Block):
     def forward(self, ctx: StepContext, x: torch.Tensor, pending, caches, next_norm: Optional[Norm] = None):
         caches = list(caches)
         conv1_cache = caches.pop(0) if self.mixer_conv is not None else None
-        mixer_cache = caches.pop(0)
+        mixer_cache = self.mixer.caches_of([caches.pop(0) for _ in self.mixer.cache_parts()])
         conv2_cache = caches.pop(0) if self.ffn_conv is not None else None
         f32_in = self.mixer.takes_float32_rows
         h = self._read(ctx, self.mixer_norm, self.mixer_conv, x, pending, conv1_cache, f32_in)
@@ -193,7 +194,7 @@ class ParallelBlock(Block):
 
     def forward(self, ctx: StepContext, x: torch.Tensor, pending, caches):
         from ..ops import kernels as K
-        cache = caches[0] if isinstance(caches, (list, tuple)) else caches
+        cache = self.mixer.caches_of(caches) if isinstance(caches, (list, tuple)) else caches
         h = self.mixer_norm.forward(x, pending)
         mark(ctx, "norm")
         d = side = None
@@ -276,7 +277,7 @@ class PostNormBlock(Block):
 
     def forward(self, ctx: StepContext, x: torch.Tensor, pending, caches):
         from ..ops import kernels as K
-        cache = caches[0] if isinstance(caches, (list, tuple)) else caches
+        cache = self.mixer.caches_of(caches) if isinstance(caches, (list, tuple)) else caches
         if isinstance(pending, NormedAhead) and pending.norm is None and pending.rows.dtype == self.rt.dtype:
             h = pending.rows                                  # the block before left the stream's rows
         else:
@@ -347,7 +348,7 @@ class OutputNormBlock(Block):
 
     def forward(self, ctx: StepContext, x: torch.Tensor, pending, caches):
         from ..ops import kernels as K
-        cache = caches[0] if isinstance(caches, (list, tuple)) else caches
+        cache = self.mixer.caches_of(caches) if isinstance(caches, (list, tuple)) else caches
         if isinstance(pending, NormedAhead) and pending.norm is None and pending.rows.dtype == self.rt.dtype:
             h = pending.rows                                  # the block before left the stream's rows
         else:

@@ -2,7 +2,7 @@
 weights: the stream and the embedding output go through one matrix together, and the pass's own
 vector is added,
 
-    x <- W_in [x ; x0] + step[t]           W_in [width, 2 width] (x first), step [times, width], t the pass
+    x <- W_in [x ; x0] [+ step[t]]         W_in [width, 2 width] (x first), step [times, width] (optional), t the pass
 
 in front of the first layer of every pass, the first pass too.  `LoopAdd` is the form without a matrix."""
 from __future__ import annotations
@@ -18,17 +18,21 @@ from .linear import Linear
 
 @register_part("loop_entry")
 class LoopEntry(Part):
-    def __init__(self, matrix: str, steps: str, width: int, times: int):
+    def __init__(self, matrix: str, steps: Optional[str], width: int, times: int):
+        """steps: the name of the passes' vectors, None for passes without."""
         self.width, self.times, self.steps_name = int(width), int(times), steps
         self.mix = Linear([matrix], 2 * self.width, [self.width], suffix="")
         self.steps: Optional[torch.Tensor] = None
 
     def tensor_specs(self) -> List[TensorSpec]:
-        return self.mix.tensor_specs() + [TensorSpec(self.steps_name, (self.times, self.width), "bias")]
+        steps = [TensorSpec(self.steps_name, (self.times, self.width), "bias")] if self.steps_name else []
+        return self.mix.tensor_specs() + steps
 
     def bind(self, get: Callable[[str], Optional[torch.Tensor]], rt: Runtime) -> None:
         super().bind(get, rt)
         self.mix.bind(get, rt)
+        if self.steps_name is None:
+            return
         self.steps = get(self.steps_name).to(device=rt.device, dtype=torch.float32).contiguous()
 
     def forward(self, ctx: StepContext, x: torch.Tensor, pending, x0: torch.Tensor, number: int):
@@ -38,7 +42,7 @@ class LoopEntry(Part):
         if isinstance(pending, (NormedAhead, K.RowSquares)):
             pending = None                         # the stream is complete already
         both = K.concat_rows(x, x0, self.rt.dtype, delta=pending, write_back=False)
-        out = K.sum_parts(self.mix.product(both, f32_ok=True), self.steps[number], torch.float32)
+        out = K.sum_parts(self.mix.product(both, f32_ok=True), None if self.steps is None else self.steps[number], torch.float32)
         return out, None
 
 

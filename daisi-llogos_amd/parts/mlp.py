@@ -56,6 +56,38 @@ class SwiGLU(FeedForward):
         return out
 
 
+@register_feed_forward("clamped_glu")
+class ClampedGLU(FeedForward):
+    """d = (g * sigmoid(1.702 g) * (u + 1)) Wd^T with g = min(x Wg^T, limit) and u = x Wu^T within -limit .. limit; no biases.
+    Gate and up are one stacked product whose row is [gate | up]."""
+    graph_safe = True
+    takes_normed_rows = True
+    adds_to_residual = True
+
+    def __init__(self, prefix: str, hidden: int, intermediate: int, limit: float, names: Sequence[str] = ("gate", "up", "down"), suffix: str = ""):
+        self.prefix, self.hidden, self.intermediate, self.limit = prefix, int(hidden), int(intermediate), float(limit)
+        self.gate_up = Linear([prefix + names[0], prefix + names[1]], hidden, [intermediate, intermediate], suffix=suffix)
+        self.down = Linear([prefix + names[2]], intermediate, [hidden], suffix=suffix)
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        return self.gate_up.tensor_specs() + self.down.tensor_specs()
+
+    def bind(self, get: Callable[[str], Optional[torch.Tensor]], rt: Runtime) -> None:
+        super().bind(get, rt)
+        self.gate_up.bind(get, rt)
+        self.down.bind(get, rt)
+
+    def forward(self, ctx: StepContext, h, residual: Optional[Residual] = None):
+        gu = self.gate_up.product(h, f32_ok=True)
+        mark(ctx, "gate_up")
+        act = K.clamped_glu(gu, self.limit, self.rt.dtype)
+        out = self.down.add_to(act, residual) if residual is not None else None
+        if out is None:
+            out = self.down.product(act, f32_ok=True)
+        mark(ctx, "down")
+        return out
+
+
 def _softplus(z: float) -> float:
     return math.log1p(math.exp(-abs(z))) + max(z, 0.0)
 

@@ -109,7 +109,10 @@ class RoutedMoE(FeedForward):
 
     Three options change the router: `scores="sigmoid"` takes the logistic function of every logit by itself, `renorm=False`
     leaves the weights as the chosen scores (times scale), `weigh="input"` puts a choice's weight on its expert's input,
-    expert_j(w_j h), instead of its output.
+    expert_j(w_j h), instead of its output; with `group_score="best_two"` a group's score is the sum of its two largest c.
+    Two change the experts: `limit` bounds their sums, expert(h) = W_down (g sigmoid(1.702 g) (u + 1)) with g = min(W_gate h,
+    limit) and u = W_up h within -limit .. limit (the shared expert then has a `shared_limit` of its own), and `out_scale` is a
+    factor on the whole output.
 
     The last `identity` router outputs have no matrices: such an expert returns h itself.  The choice, the
     sorting of the (token, choice) pairs by expert and the weighted sum are made on the device, so single-token
@@ -132,7 +135,8 @@ class RoutedMoE(FeedForward):
 
     def __init__(self, prefix: str, hidden: int, n_experts: int, top: int, intermediate: int, identity: int = 0,
                  groups: int = 1, keep: int = 1, scale: float = 1.0, shared_intermediate: int = 0, correction: bool = True,
-                 scores: str = "softmax", renorm: bool = True, weigh: str = "output"):
+                 scores: str = "softmax", renorm: bool = True, weigh: str = "output", group_score: str = "best",
+                 limit: Optional[float] = None, shared_limit: Optional[float] = None, out_scale: float = 1.0):
         total = int(n_experts) + int(identity)
         if not 1 <= top <= total <= K.MOE_MAX_EXPERTS:
             raise ValueError(f"top {top} of {total} router outputs: outside 1..outputs..{K.MOE_MAX_EXPERTS}")
@@ -142,7 +146,13 @@ class RoutedMoE(FeedForward):
             raise ValueError(f"{groups} groups of which {keep} are kept do not fit {total} router outputs and top {top}")
         if scores not in ("softmax", "sigmoid") or weigh not in ("output", "input"):
             raise ValueError(f"scores '{scores}' (softmax, sigmoid), weigh '{weigh}' (output, input)")
-        self.scores, self.renorm, self.weigh = scores, bool(renorm), weigh
+        if group_score not in ("best", "best_two"):
+            raise ValueError(f"group_score '{group_score}' (best, best_two)")
+        if out_scale != 1.0 and weigh == "input":
+            raise ValueError("a factor on the output is not built beside weights on the experts' inputs")
+        self.scores, self.renorm, self.weigh, self.group_score = scores, bool(renorm), weigh, group_score
+        self.limit = None if limit is None else float(limit)
+        self.out_scale = float(out_scale)
         self.prefix, self.hidden = prefix, int(hidden)
         self.n_experts, self.identity, self.top, self.intermediate = int(n_experts), int(identity), int(top), int(intermediate)
         self.groups, self.keep, self.scale = int(groups), int(keep), float(scale)
@@ -151,8 +161,9 @@ class RoutedMoE(FeedForward):
         self.shared = None
         self.probed = None          # {"choice": int32 [T, top]} of the last step that was run part by part (measurements)
         if self.shared_intermediate:
-            from .mlp import SwiGLU
-            self.shared = SwiGLU(prefix + "shared.", hidden, self.shared_intermediate, names=("gate", "up", "down"), suffix="")
+            from .mlp import ClampedGLU, SwiGLU
+            own = dict(prefix=prefix + "shared.", hidden=hidden, intermediate=self.shared_intermediate, names=("gate", "up", "down"), suffix="")
+            self.shared = SwiGLU(**own) if shared_limit is None else ClampedGLU(limit=shared_limit, **own)
 
     @property
     def outputs(self) -> int:
@@ -202,8 +213,8 @@ class RoutedMoE(FeedForward):
             side.wait_stream(main)                       # h is there
             with torch.cuda.stream(side):
                 shared = _float32(self.shared.forward(ctx, h))
-        choice, weight = K.moe_router(h, self.router_w, self.correction, self.groups, self.keep, self.top, self.scale,
-                                      scores=self.scores, renorm=self.renorm)
+        choice, weight = K.moe_router(h, self.router_w, self.correction, self.groups, self.keep, self.top,
+                                      self.scale * self.out_scale, scores=self.scores, renorm=self.renorm, group_score=self.group_score)
         mark(ctx, "router")
         if ctx is not None and ctx.probe is not None:
             self.probed = {"choice": choice}
@@ -211,7 +222,7 @@ class RoutedMoE(FeedForward):
         if self.n_experts:
             order, seg, where = K.moe_route(None, choice, self.outputs)
             act = K.moe_product(h, self.gate_up, order, seg, self.top, True, self.rt.dtype, gated=True,
-                                pair_weight=weight.view(-1) if self.weigh == "input" else None)
+                                pair_weight=weight.view(-1) if self.weigh == "input" else None, limit=self.limit)
             y = K.moe_product(act, self.down, order, seg, self.top, False, torch.float32)
         else:
             where = torch.zeros(T * self.top, dtype=torch.int32, device=h.device)
@@ -225,7 +236,7 @@ class RoutedMoE(FeedForward):
         x = residual.x if residual is not None else None
         rows = x is not None and residual.norm is not None and residual.norm.plain_rows
         out = K.moe_combine_weighted(y, where, choice, weight if self.weigh == "output" else None, self.n_experts, h, shared,
-                                     stream=x, rows=rows and not self.rt.is_f32)
+                                     stream=x, rows=rows and not self.rt.is_f32, shared_scale=self.out_scale)
         mark(ctx, "combine")
         # (added to the stream: what is left is its rows, for a reader that takes them as they are)
         return out if x is None else K.RowSquares(None, W, out, residual.norm.row_weight() if rows else None)
