@@ -240,6 +240,27 @@ def peponex_config(width, runs, vocab, ff):
             "token_side": {"dim": 256}, "loop": {"start": 1, "stop": 3, "times": 2}, "layers": layers, "torch_dtype": "bfloat16"}
 
 
+def zisedra_config(width, runs, vocab, ff):
+    """Layers of real sizes: a recurrence by the gated delta rule in front and behind, between them window attention beside
+    such a recurrence, the first two of those gone through twice, which makes `runs` runs of `runs - 2` layers.  Heads of
+    128 key and value channels throughout: recurrences with half as many key heads as value heads (alone) and as many
+    (beside attention, decay and gate of rank width / 16), four taps; attention with four query heads a key/value head,
+    half of a head rotated, a window of 1,024; mixtures of 16 experts in 4 groups of which 2 are kept, 2 a token, each
+    expert a quarter and the shared one half as wide as the dense decoder's feed-forward (the dense decoder's matrix
+    bytes a token)."""
+    heads = width // 128
+    moe = {"kind": "moe", "expert": {"ff": ff // 4, "limit": 7.0}, "shared": {"ff": ff // 2, "limit": 7.0},
+           "router": {"experts": 16, "top": 2, "groups": {"count": 4, "keep": 2}}}
+    rec = {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4}
+    att = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 1024},
+           "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    alone = {"type": "delta", "mixer": rec, "mlp": moe}
+    both = {"type": "parallel", "mixer": {"left": att, "right": dict(rec, kv_heads=heads)}, "mlp": moe}
+    n = runs - 2
+    return {"architecture": "Zisedra", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "residual_mult": 0.5,
+            "loop": {"start": 1, "stop": 3, "times": 2}, "layers": [alone] + [both] * (n - 2) + [alone], "torch_dtype": "bfloat16"}
+
+
 def moe_bytes_read(model, ids) -> int:
     """Bytes of weights that a step with the token ids `ids` reads: as step_weight_bytes, but of a layer's experts
     only those that the layer's table names for these ids, or that its router chose in the last step that was
@@ -306,7 +327,7 @@ def compare_designs(args) -> int:
             eng.step([(x, toks(args.prompt_len)) for x in slots], want="last")
             ids = toks(batch)                                     # a token of its own for every sequence (an expert choice of its own)
             step = lambda: eng.step([(x, [t]) for x, t in zip(slots, ids)], want="last", borrow=True)
-            if label.split()[0] in ("zasidra", "peponex"):
+            if label.split()[0] in ("zasidra", "peponex", "zisedra"):
                 # a step run part by part leaves every router's choice behind: the experts that such a step reads
                 eng.step([(x, [t]) for x, t in zip(slots, ids)], want="last", probe=llogos.StepProbe())
             for _ in range(args.warmup):
@@ -334,6 +355,8 @@ def compare_designs(args) -> int:
                      num_attention_heads=width // 128, num_key_value_heads=max(1, width // 512), tie_word_embeddings=True)
         if args.design == "zogurax":
             other = zogurax_config(width, layers, vocab, ff)
+        elif args.design == "zisedra":
+            other = zisedra_config(width, layers, vocab, ff)
         elif args.design == "peponex":
             other = peponex_config(width, layers, vocab, ff)
         elif args.design == "zasidra":
@@ -347,6 +370,9 @@ def compare_designs(args) -> int:
         if args.design in ("batodra", "peponex"):
             # the other design that mixes recurrent layers with attention, at the same sizes
             entry["nipulorn"] = measure(f"nipulorn {name}", nipulorn_config(width, layers, vocab, ff * 3 // 2), vocab)
+        if args.design == "zisedra":
+            # the other design that mixes matrix-state recurrences, window attention and routed experts
+            entry["peponex"] = measure(f"peponex {name}", peponex_config(width, layers, vocab, ff), vocab)
         if args.design == "zasidra":
             # the other design with attention behind a norm over the whole projection and a mixture of experts
             entry["zogurax"] = measure(f"zogurax {name}", zogurax_config(width, layers, vocab, ff), vocab)
@@ -358,7 +384,7 @@ def compare_designs(args) -> int:
 
 def main(argv=None) -> int:
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["nipulorn", "zogurax", "batodra", "zasidra", "peponex"], default=None,
+    ap.add_argument("--design", choices=["nipulorn", "zogurax", "batodra", "zasidra", "peponex", "zisedra"], default=None,
                     help="instead of the default run: this design beside the dense decoder at equal sizes (prefill, decode, parts)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=248)   # + 8 warm-up = 256 new tokens

@@ -92,10 +92,13 @@ __device__ __forceinline__ float delta_input(const DeltaRows& r, const float* ri
 // One block a (sequence, head).  Thread (p, x) holds VEC neighbouring columns of rows p, p + P, ... of S in registers from
 // the first load to the store; both column sums S^T k and S^T q come from one pass, since with k . q known
 // o = (g S)^T q + (k . q) u.
-template <int VEC, int RPT, typename TO>
-__global__ __launch_bounds__(1024) void delta_step_kernel(TO* __restrict__ y, DeltaRows in, DeltaGates gt, const float* __restrict__ gate,
-                                                          int ldg, int gate_parts, size_t gate_part_stride, int gate_silu,
-                                                          const float* __restrict__ norm_w, float eps) {
+// A block's time is the latency of its loads, so all that a thread needs (its share of S, a channel of q, of k and of v with
+// the rows before them, its decay, beta, the gate) is asked for before the first sum; up to four taps and four parts of
+// a product that way (TAPS 4), more in loops.
+template <int VEC, int RPT, int NT, int TAPS, typename TO>
+__global__ __launch_bounds__(NT) void delta_step_kernel(TO* __restrict__ y, DeltaRows in, DeltaGates gt, const float* __restrict__ gate,
+                                                        int ldg, int gate_parts, size_t gate_part_stride, int gate_silu,
+                                                        const float* __restrict__ norm_w, float eps) {
     extern __shared__ float lds[];
     __shared__ float red[3][16];
     const int D = in.D, V = in.V, H = in.H, G = in.G;
@@ -103,7 +106,9 @@ __global__ __launch_bounds__(1024) void delta_step_kernel(TO* __restrict__ y, De
     float* sq = lds;                       // [D]
     float* sk = sq + D;                    // [D]
     float* sg = sk + D;                    // [D]
-    float* su = sg + D;                    // [width VEC]
+    float* sv = sg + D;                    // [V]
+    float* sz = sv + V;                    // [V] the gate's logits
+    float* su = sz + V;                    // [width VEC]
     float* sum = su + width * VEC;         // [2][P][width VEC]
     const int seq = blockIdx.x, head = blockIdx.y, kvh = head / (H / G);
     const int tid = threadIdx.x, p = tid / width, c0 = (tid % width) * VEC;
@@ -112,6 +117,7 @@ __global__ __launch_bounds__(1024) void delta_step_kernel(TO* __restrict__ y, De
     float* slot = in.state + (size_t)in.slots[seq] * in.state_stride;
     float* ring = slot + in.ring;
     float* S = slot + (size_t)head * D * V + c0;
+    const int turn = pos % in.taps;        // the ring's row of this position
 
     float s[RPT][VEC];
 #pragma unroll
@@ -129,33 +135,79 @@ __global__ __launch_bounds__(1024) void delta_step_kernel(TO* __restrict__ y, De
             for (int e = 0; e < VEC; ++e) s[r][e] = 0.f;
         }
     }
-    // a channel of the token through the convolution and silu; its raw value joins the ring (`keep`)
-    auto channel = [&](int c, bool keep) {
-        const float x0 = delta_sum_parts(in.rows + (size_t)seq * in.ld + c, in.parts, in.part_stride);
-        float acc = x0 * in.conv[(size_t)(in.taps - 1) * in.W + c];
-#pragma unroll 4
-        for (int j = 1; j < in.taps; ++j)
-            if (pos >= j) acc = fmaf(in.conv[(size_t)(in.taps - 1 - j) * in.W + c], ring[(size_t)((pos - j) % in.taps) * in.W + c], acc);
-        if (keep) ring[(size_t)(pos % in.taps) * in.W + c] = x0;
-        return delta_silu(acc);
+    // the threads take channels of q and k from the front and of v from the back (D and V are at most blockDim)
+    const int d = min(tid, D - 1), vi = (int)blockDim.x - 1 - tid, v_at = min(vi, V - 1);
+    const bool has_k = tid < D, has_v = vi < V;
+    const int chan[3] = {kvh * D + d, (G + kvh) * D + d, 2 * G * D + head * V + v_at};
+    const float* row = in.rows + (size_t)seq * in.ld;
+    const int zc = gt.channelwise ? head * D + d : head;
+    const float* zp = gt.z + (size_t)seq * gt.ldz + zc;
+    const float* gp = gate + (size_t)seq * ldg + head * V + v_at;
+    const float* bp = row + gt.b_col + head;
+    auto ask = [](const float* q, int parts, size_t stride, float (&to)[4]) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) to[j] = q[(size_t)min(j, parts - 1) * stride];
     };
-    const float beta = delta_sigmoid(delta_sum_parts(in.rows + (size_t)seq * in.ld + gt.b_col + head, in.parts, in.part_stride));
-    const float a_log = gt.a_log[head];
-    const bool first = head % (H / G) == 0;
-    float qq = 0.f, kk = 0.f, qk = 0.f;
-    for (int d = tid; d < D; d += blockDim.x) {
-        const float q = channel(kvh * D + d, first), k = channel((G + kvh) * D + d, first);
-        const int zc = gt.channelwise ? head * D + d : head;
-        const float z = delta_sum_parts(gt.z + (size_t)seq * gt.ldz + zc, gt.z_parts, gt.z_part_stride) + gt.dt_bias[zc];
-        sq[d] = q;
-        sk[d] = k;
-        sg[d] = delta_exp2(delta_log_decay(z, a_log));
-        qq = fmaf(q, q, qq); kk = fmaf(k, k, kk); qk = fmaf(q, k, qk);
+    auto total = [](const float* q, int parts, size_t stride, const float (&from)[4]) {
+        float v = from[0];
+#pragma unroll
+        for (int j = 1; j < 4; ++j) v += j < parts ? from[j] : 0.f;
+        for (int j = 4; j < parts; ++j) v += q[(size_t)j * stride];
+        return v;
+    };
+    float raw[3], act[3], z, z_out, b_logit;
+    const float dt_bias = gt.dt_bias[zc], a_log = gt.a_log[head];
+    if (TAPS == 4) {
+        float x0[3][4], xs[3][4], w[3][4], zq[4], gq[4], bq[4];
+#pragma unroll
+        for (int i = 0; i < 3; ++i) {
+            ask(row + chan[i], in.parts, in.part_stride, x0[i]);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {                  // the row `j` positions back and its tap
+                const int back = min(j, in.taps - 1), at = turn - back + (turn < back ? in.taps : 0);
+                w[i][j] = in.conv[(size_t)(in.taps - 1 - back) * in.W + chan[i]];
+                xs[i][j] = j > 0 ? ring[(size_t)at * in.W + chan[i]] : 0.f;
+            }
+        }
+        ask(zp, gt.z_parts, gt.z_part_stride, zq);
+        ask(gp, gate_parts, gate_part_stride, gq);
+        ask(bp, in.parts, in.part_stride, bq);
+#pragma unroll
+        for (int i = 0; i < 3; ++i) {
+            raw[i] = total(row + chan[i], in.parts, in.part_stride, x0[i]);
+            float acc = raw[i] * w[i][0];
+#pragma unroll
+            for (int j = 1; j < 4; ++j) acc = fmaf(w[i][j], (j < in.taps && pos >= j) ? xs[i][j] : 0.f, acc);
+            act[i] = delta_silu(acc);
+        }
+        z = total(zp, gt.z_parts, gt.z_part_stride, zq);
+        z_out = total(gp, gate_parts, gate_part_stride, gq);
+        b_logit = total(bp, in.parts, in.part_stride, bq);
+    } else {
+#pragma unroll
+        for (int i = 0; i < 3; ++i) {
+            raw[i] = delta_sum_parts(row + chan[i], in.parts, in.part_stride);
+            float acc = raw[i] * in.conv[(size_t)(in.taps - 1) * in.W + chan[i]];
+            for (int j = 1; j < in.taps; ++j)
+                if (pos >= j) acc = fmaf(in.conv[(size_t)(in.taps - 1 - j) * in.W + chan[i]],
+                                         ring[(size_t)(turn - j + (turn < j ? in.taps : 0)) * in.W + chan[i]], acc);
+            act[i] = delta_silu(acc);
+        }
+        z = delta_sum_parts(zp, gt.z_parts, gt.z_part_stride);
+        z_out = delta_sum_parts(gp, gate_parts, gate_part_stride);
+        b_logit = delta_sum_parts(bp, in.parts, in.part_stride);
     }
-    float v = 0.f, z_out = 0.f;
-    if (tid < V) {
-        v = channel(2 * G * D + head * V + tid, true);
-        z_out = delta_sum_parts(gate + (size_t)seq * ldg + head * V + tid, gate_parts, gate_part_stride);
+    const float beta = delta_sigmoid(b_logit);
+    float qq = 0.f, kk = 0.f, qk = 0.f;
+    if (has_k) {
+        sq[d] = act[0];
+        sk[d] = act[1];
+        sg[d] = delta_exp2(delta_log_decay(z + dt_bias, a_log));
+        qq = act[0] * act[0]; kk = act[1] * act[1]; qk = act[0] * act[1];
+    }
+    if (has_v) {
+        sv[vi] = act[2];
+        sz[vi] = z_out;
     }
     qq = wave_sum(qq); kk = wave_sum(kk); qk = wave_sum(qk);
     const int lane = tid & (kWave - 1), wave = tid / kWave, nwaves = blockDim.x / kWave;
@@ -196,13 +248,19 @@ __global__ __launch_bounds__(1024) void delta_step_kernel(TO* __restrict__ y, De
             rk += sum[(size_t)w * width * VEC + tid];
             rq += sum[(size_t)(P + w) * width * VEC + tid];
         }
-        const float u = beta * (v - ks * rk);
+        const float u = beta * (sv[tid] - ks * rk);
         su[tid] = ks * u;
         o = fmaf(kq, u, qs * rq);
     }
     const float inv = 1.0f / sqrtf(block_sum(o * o, red[0]) / (float)V + eps);      // (its barriers also publish su)
     if (tid < V)
-        store_f32(y + ((size_t)seq * H + head) * V + tid, o * inv * norm_w[tid] * (gate_silu ? delta_silu(z_out) : delta_sigmoid(z_out)));
+        store_f32(y + ((size_t)seq * H + head) * V + tid, o * inv * norm_w[tid] * (gate_silu ? delta_silu(sz[tid]) : delta_sigmoid(sz[tid])));
+    // the token's projected channels join the ring (those of a key head once)
+    if (has_k && head % (H / G) == 0) {
+        ring[(size_t)turn * in.W + chan[0]] = raw[0];
+        ring[(size_t)turn * in.W + chan[1]] = raw[1];
+    }
+    if (has_v) ring[(size_t)turn * in.W + chan[2]] = raw[2];
 #pragma unroll
     for (int r = 0; r < RPT; ++r) {
         const int d = p + r * P;
@@ -227,7 +285,7 @@ static bool delta_rows_ok(int ld, int parts, int taps, long long state_stride, i
 static int delta_step_threads(int D, int V, int vec) {
     const int width = (V + vec - 1) / vec;
     for (int t = 256; t <= 1024; t *= 2) {
-        if (t < V || t < width) continue;
+        if (t < V) continue;
         const int P = t / width;
         if ((D + P - 1) / P * vec <= 64) return t;
     }
@@ -255,17 +313,21 @@ LLOGOS_EXPORT int llogos_delta_step(void* y, int y_dtype, const float* rows, int
     const int per = vec ? 4 : 1, threads = delta_step_threads(D, V, per);
     if (!threads) return LLOGOS_UNSUPPORTED;
     const int width = (V + per - 1) / per, P = threads / width, rpt = (D + P - 1) / P;
-    const size_t smem = (size_t)(3 * D + width * per * (1 + 2 * P)) * sizeof(float);
+    const size_t smem = (size_t)(3 * D + 2 * V + width * per * (1 + 2 * P)) * sizeof(float);
     if (smem > 64 * 1024) return LLOGOS_UNSUPPORTED;
-#define DS(VEC_, RPT_, TO) delta_step_kernel<VEC_, RPT_, TO><<<dim3(B, H), threads, smem, stream>>>((TO*)y, in, gt, gate, ldg, gate_parts, \
-        (size_t)gate_part_stride, gate_silu, norm_w, eps)
+#define DS(VEC_, RPT_, NT, TAPS, TO) delta_step_kernel<VEC_, RPT_, NT, TAPS, TO><<<dim3(B, H), threads, smem, stream>>>((TO*)y, in, gt, \
+        gate, ldg, gate_parts, (size_t)gate_part_stride, gate_silu, norm_w, eps)
+#define DSV(NT, TAPS, TO) do { if (rpt <= 4) DS(4, 4, NT, TAPS, TO); else if (rpt <= 8) DS(4, 8, NT, TAPS, TO); else DS(4, 16, NT, TAPS, TO); } while (0)
 #define DSR(TO) do { \
-        if (vec) { if (rpt <= 4) DS(4, 4, TO); else if (rpt <= 8) DS(4, 8, TO); else DS(4, 16, TO); } \
-        else { if (rpt <= 16) DS(1, 16, TO); else DS(1, 64, TO); } } while (0)
+        if (!vec) { if (rpt <= 16) DS(1, 16, 1024, 16, TO); else DS(1, 64, 1024, 16, TO); } \
+        else if (taps > 4 || threads > 512) DSV(1024, 16, TO); \
+        else if (threads == 256) DSV(256, 4, TO); \
+        else DSV(512, 4, TO); } while (0)
     if (y_dtype == DT_F32) DSR(float);
     else if (y_dtype == DT_BF16) DSR(bf16_t);
     else return LLOGOS_BAD_ARGUMENT;
 #undef DSR
+#undef DSV
 #undef DS
     return LLOGOS_LAUNCH_CHECK();
 }

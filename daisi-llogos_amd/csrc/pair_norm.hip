@@ -5,7 +5,7 @@
 // sum v itself is left in `delta`, float [T, H].  A factor on the sum belongs into wa and wb.  All arithmetic is 32-bit.
 #include "common.h"
 
-constexpr int kPairParts = 4;          // parts of a product whose loads are in flight together
+constexpr int kPairParts = 8;          // parts of a product whose loads are in flight together
 
 // One block a row; a thread keeps its ITEMS values of the row in registers from pass to pass.
 template <typename TA, typename TB, typename TH, int ITEMS>

@@ -151,7 +151,7 @@ def window_attention(h, t, m: dict) -> np.ndarray:
     out = np.zeros((T, H, V))
     for head in range(H):
         kv = head // (H // G)
-        out[:, head] = window_softmax((q[:, head] @ k[:, kv].T) * m["scale"], m["mask"]["size"]) @ v[:, kv]
+        out[:, head] = window_softmax((q[:, head] @ k[:, kv].T) * m["scale"], m["mask"]["size"] if m.get("mask") else T) @ v[:, kv]
     return out.reshape(T, H * V) @ t["o"].T
 
 
@@ -229,6 +229,15 @@ def forward(cfg: dict, w: dict, tokens, layers=None) -> np.ndarray:
         if layers is not None:
             layers.append(x.copy())
     return norm(x, w["final.norm"], eps) @ w["embed"].T
+
+
+def generate_greedy(cfg: dict, w: dict, prompt, n: int) -> list:
+    """n tokens, each the first largest logit after everything before it (the whole sequence is run again each time)."""
+    seq, out = list(prompt), []
+    for _ in range(n):
+        out.append(int(np.argmax(forward(cfg, w, seq)[-1])))
+        seq.append(out[-1])
+    return out
 
 
 def load(folder: str):
