@@ -68,7 +68,7 @@ __global__ void concat_rows_kernel(TO* __restrict__ out, float* __restrict__ a, 
                                    size_t part_stride, const float* __restrict__ b, int Wa, int Wb, int write_back) {
     const int t = blockIdx.x;
     TO* o = out + (size_t)t * (Wa + Wb);
-    for (int i = threadIdx.x; i < Wa + Wb; i += blockDim.x) {
+    for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < Wa + Wb; i += gridDim.y * blockDim.x) {
         float v;
         if (i < Wa) {
             v = a[(size_t)t * Wa + i];
@@ -86,10 +86,13 @@ __global__ void concat_rows_kernel(TO* __restrict__ out, float* __restrict__ a, 
 LLOGOS_EXPORT int llogos_concat_rows(void* out, int out_dtype, float* a, const float* delta, int parts, long long part_stride,
                                      const float* b, int T, int Wa, int Wb, int write_back, hipStream_t stream) {
     if (T <= 0 || Wa <= 0 || Wb <= 0 || parts < 1) return LLOGOS_BAD_ARGUMENT;
+    // few rows: a value a thread, so that a row's loads are all on their way at once; many: four blocks a row
+    const int all = (Wa + Wb + 255) / 256;
+    const dim3 grid(T, T <= 64 || all < 4 ? all : 4);
     if (out_dtype == DT_F32)
-        concat_rows_kernel<float><<<T, 256, 0, stream>>>((float*)out, a, delta, parts, (size_t)part_stride, b, Wa, Wb, write_back);
+        concat_rows_kernel<float><<<grid, 256, 0, stream>>>((float*)out, a, delta, parts, (size_t)part_stride, b, Wa, Wb, write_back);
     else if (out_dtype == DT_BF16)
-        concat_rows_kernel<bf16_t><<<T, 256, 0, stream>>>((bf16_t*)out, a, delta, parts, (size_t)part_stride, b, Wa, Wb, write_back);
+        concat_rows_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)out, a, delta, parts, (size_t)part_stride, b, Wa, Wb, write_back);
     else
         return LLOGOS_BAD_ARGUMENT;
     return LLOGOS_LAUNCH_CHECK();

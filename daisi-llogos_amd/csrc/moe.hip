@@ -255,6 +255,7 @@ __global__ __launch_bounds__(256) void moe_router_logits_kernel(float* __restric
     for (int r = 0; r < R; ++r)
 #pragma unroll
         for (int g = 0; g < G; ++g) acc[r][g] = 0.f;
+#pragma unroll (R == 1 ? 8 : 1)                              // (few rows: a wave alone on its unit waits for every load)
     for (int k = 4 * lane; k < K; k += 4 * kWave) {
         float4 av[R], wv[G];
 #pragma unroll
@@ -296,14 +297,14 @@ LLOGOS_EXPORT int llogos_moe_router_logits(float* z, const void* a, int a_dtype,
     if (T <= 0 || E <= 0 || K <= 0 || lda < K || (a_dtype != DT_F32 && a_dtype != DT_BF16)) return LLOGOS_BAD_ARGUMENT;
     const int elt = a_dtype == DT_F32 ? 4 : 2;
     const bool vec = K % 4 == 0 && lda % 4 == 0 && (uintptr_t)a % (4 * elt) == 0 && (uintptr_t)w % 16 == 0;
-    // few rows: a row a wave and four outputs, so that the step has waves enough; many: four rows a wave and eight outputs
+    // few rows: a row a wave and one output, so that the step has waves enough; many: four rows a wave and eight outputs
     const bool few = T <= 64;
-    const int R = few ? 1 : 4, G = few ? 4 : 8;
+    const int R = few ? 1 : 4, G = few ? 1 : 8;
     dim3 grid((T + 4 * R - 1) / (4 * R), (E + G - 1) / G);
 #define RL(TA, R_, G_, V) moe_router_logits_kernel<TA, R_, G_, V><<<grid, 256, 0, stream>>>(z, (const TA*)a, lda, w, T, E, K)
 #define RLV(TA, R_, G_) do { if (vec) RL(TA, R_, G_, true); else RL(TA, R_, G_, false); } while (0)
-    if (a_dtype == DT_F32) { if (few) RLV(float, 1, 4); else RLV(float, 4, 8); }
-    else { if (few) RLV(bf16_t, 1, 4); else RLV(bf16_t, 4, 8); }
+    if (a_dtype == DT_F32) { if (few) RLV(float, 1, 1); else RLV(float, 4, 8); }
+    else { if (few) RLV(bf16_t, 1, 1); else RLV(bf16_t, 4, 8); }
 #undef RLV
 #undef RL
     return LLOGOS_LAUNCH_CHECK();

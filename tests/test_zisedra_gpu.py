@@ -555,6 +555,25 @@ def test_two_mixers_side_by_side_alone_in_pieces(hidden, kind, dtype):
             assert isinstance(left_over, K.RowSquares) and left_over.unscaled is None
 
 
+@pytest.mark.parametrize("dtype", H.DTYPES)
+@pytest.mark.parametrize("name", ["zis_a", "zis_c"])
+def test_the_second_stream_changes_no_bit(name, dtype, monkeypatch):
+    """Replayed and launched, whether the left mixer runs beside the right one or in front of it."""
+    outs = []
+    monkeypatch.setattr(P.SideBySide, "side_bytes", 0)
+    for rows in (64, 0):
+        monkeypatch.setattr(P.SideBySide, "side_rows", rows)
+        for graphs in (True, False):
+            eng = H.engine(name, dtype, use_graphs=graphs)
+            a, b = eng.alloc_slot(), eng.alloc_slot()
+            toks = H.tokens(name, 140, 13)
+            got = [_np(eng.step([(a, list(toks[:60])), (b, list(toks[70:75]))], want="all"))]
+            for t in range(60):
+                got.append(_np(eng.step([(a, [toks[60 + t]]), (b, [toks[75 + t]])], want="all")))
+            outs.append(np.concatenate(got))
+    assert all(np.array_equal(o, outs[0]) for o in outs[1:])
+
+
 @pytest.mark.parametrize("block", ["pre_norm", "sandwich", "parallel", "post_norm", "output_norm"])
 def test_every_block_hands_a_pair_of_mixers_their_own_caches(block):
     """A mixer made of two asks the cache for two units, in whatever block it stands."""
