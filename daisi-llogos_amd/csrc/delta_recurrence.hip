@@ -463,6 +463,14 @@ LLOGOS_EXPORT int llogos_delta_prepare(float* act, float* logd, float* beta, con
 //   [2][DTP] -T K'   [2][DTP] q exp(b) - M K'   [DTP][2] (k exp(b_n - b))^T   [2][VTN] T V' (laid out as a result)   [16 DTP] exp(b_n)
 __host__ __device__ __forceinline__ size_t delta_chunk_floats(int DTP, int VTN) { return (size_t)256 * (6 * DTP + 2 * VTN) + 16 * DTP; }
 
+// A barrier for what the block's waves exchange through LDS alone: loads from memory that are on their way, and stores,
+// are not waited for (__syncthreads waits for all of them, and with them for everything asked for ahead).
+__device__ __forceinline__ void delta_lds_barrier() {
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+}
+
 __device__ __forceinline__ dl4 delta_mfma4(dl4 a, dl4 b, dl4 acc) {
 #pragma unroll
     for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], b[e], acc, 0, 0, 0);
@@ -514,6 +522,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(float* __restrict__ ws
     float* out = ws + ((size_t)blockIdx.x * H + head) * delta_chunk_floats(DTP, VTN);
 
     if (tid < C) s_beta[tid] = tid < n ? beta[(size_t)(first + tid) * H + head] : 0.f;
+#pragma unroll 4
     for (int e = tid; e < C * 4 * DTP; e += 256) {
         const int j = e / (4 * DTP), d = 4 * (e % (4 * DTP));
         dl4 q = {0.f, 0.f, 0.f, 0.f}, k = q;
@@ -553,7 +562,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(float* __restrict__ ws
         }
         if (lane < C) s_b[lane] = x;
     }
-    __syncthreads();
+    delta_lds_barrier();
     // the logarithm's sum within row j's run of 16, channel d .. d + 3
     auto rel4 = [&](int j, int d) {
         if (CHANNELWISE) return delta_ld4(sB + j * DP + d);
@@ -583,26 +592,61 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(float* __restrict__ ws
             }
         }
     } else {
-        // the tiles on the diagonal pair by pair: the decays' quotients differ from channel to channel
+        // the tiles on the diagonal pair by pair: the decays' quotients differ from channel to channel.  A wave takes a tile
+        // and half of the channels, a lane 2 x 2 pairs; the halves meet in LDS.
+        {
+            const int it = wave >> 1, half = wave & 1, i0 = 16 * it + 2 * (lane >> 3), j0 = 16 * it + 2 * (lane & 7);
+            const int mid = 8 * DTP, d_end = half ? min(16 * DTP, (D + 3) & ~3) : min(mid, (D + 3) & ~3);        // (channels behind D hold zeros)
+            float kk[2][2] = {{0.f, 0.f}, {0.f, 0.f}}, qk[2][2] = {{0.f, 0.f}, {0.f, 0.f}};
+            if (j0 <= i0 + 1) {
+                for (int d = half ? mid : 0; d < d_end; d += 4) {
+                    dl4 ki[2], qi[2], bi[2], kj[2], bj[2];
 #pragma unroll
-        for (int it = 0; it < 2; ++it) {
-            const int i = 16 * it + 4 * (it ? 3 - wave : wave) + g, j = 16 * it + c;
-            float kk = 0.f, qk = 0.f;
-            if (j <= i) {
-                for (int d = 0; d < D; d += 4) {           // (channels behind D hold zeros)
-                    const dl4 ki = delta_ld4(sK + i * DP + d), qi = delta_ld4(sQ + i * DP + d), kj = delta_ld4(sK + j * DP + d);
-                    const dl4 x = kj * delta_exp2(delta_ld4(sB + i * DP + d) - delta_ld4(sB + j * DP + d));
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) {
-                        kk = fmaf(ki[e], x[e], kk);
-                        qk = fmaf(qi[e], x[e], qk);
+                    for (int a = 0; a < 2; ++a) {
+                        ki[a] = delta_ld4(sK + (i0 + a) * DP + d);
+                        qi[a] = delta_ld4(sQ + (i0 + a) * DP + d);
+                        bi[a] = delta_ld4(sB + (i0 + a) * DP + d);
+                        kj[a] = delta_ld4(sK + (j0 + a) * DP + d);
+                        bj[a] = delta_ld4(sB + (j0 + a) * DP + d);
                     }
+#pragma unroll
+                    for (int a = 0; a < 2; ++a)
+#pragma unroll
+                        for (int b = 0; b < 2; ++b) {
+                            // (a pair above the diagonal is not used; its exponent would be positive)
+                            const dl4 x = kj[b] * delta_exp2(j0 + b <= i0 + a ? bi[a] - bj[b] : dl4{0.f, 0.f, 0.f, 0.f});
+#pragma unroll
+                            for (int e = 0; e < 4; ++e) {
+                                kk[a][b] = fmaf(ki[a][e], x[e], kk[a][b]);
+                                qk[a][b] = fmaf(qi[a][e], x[e], qk[a][b]);
+                            }
+                        }
                 }
             }
-            sA[i * CP + j] = j < i ? s_beta[i] * kk : 0.f;
-            sP[i * CP + j] = qk;
+            float* hA = sT + it * 16 * CP;                 // (T and M are not there yet)
+            float* hP = sM + it * 16 * CP;
+            if (half) {
+#pragma unroll
+                for (int a = 0; a < 2; ++a)
+#pragma unroll
+                    for (int b = 0; b < 2; ++b) {
+                        hA[(i0 + a - 16 * it) * CP + j0 + b - 16 * it] = kk[a][b];
+                        hP[(i0 + a - 16 * it) * CP + j0 + b - 16 * it] = qk[a][b];
+                    }
+            }
+            delta_lds_barrier();
+            if (!half) {
+#pragma unroll
+                for (int a = 0; a < 2; ++a)
+#pragma unroll
+                    for (int b = 0; b < 2; ++b) {
+                        const int i = i0 + a, j = j0 + b;
+                        sA[i * CP + j] = j < i ? s_beta[i] * (kk[a][b] + hA[(i - 16 * it) * CP + j - 16 * it]) : 0.f;
+                        sP[i * CP + j] = j <= i ? qk[a][b] + hP[(i - 16 * it) * CP + j - 16 * it] : 0.f;
+                    }
+            }
         }
-        if (wave == 0) {
+        if (wave == 1) {                                   // (the waves of the halves have less to do at the end)
             dl4 kk = {0.f, 0.f, 0.f, 0.f}, qk = kk;
             for (int dt = 0; dt < DTP; ++dt) {
                 const int d = 16 * dt + 4 * g;
@@ -619,7 +663,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(float* __restrict__ ws
             }
         }
     }
-    __syncthreads();
+    delta_lds_barrier();
     // ---- T = (I + A)^-1: the diagonal tiles column by column, the tile below from them
     if (wave < 2) {
         const float* a = sA + 16 * wave * CP + 16 * wave;
@@ -636,7 +680,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(float* __restrict__ ws
             for (int i = 0; i < 16; ++i) sT[(16 * wave + i) * CP + 16 * wave + c] = x[i];
         }
     }
-    __syncthreads();
+    delta_lds_barrier();
     auto column4 = [&](const float* m, int r0, int col) {  // rows r0 .. r0 + 3 of a column of a [32][36] matrix
         return dl4{m[r0 * CP + col], m[(r0 + 1) * CP + col], m[(r0 + 2) * CP + col], m[(r0 + 3) * CP + col]};
     };
@@ -647,7 +691,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(float* __restrict__ ws
 #pragma unroll
         for (int r = 0; r < 4; ++r) sT[(16 + 4 * g + r) * CP + c] = -t[r];
     }
-    __syncthreads();
+    delta_lds_barrier();
     // ---- M = P T
     if (wave < 3) {
         const int it = wave > 0 ? 1 : 0, jt = wave > 1 ? 1 : 0;
@@ -657,7 +701,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(float* __restrict__ ws
 #pragma unroll
         for (int r = 0; r < 4; ++r) sM[(16 * it + 4 * g + r) * CP + 16 * jt + c] = m[r];
     }
-    __syncthreads();
+    delta_lds_barrier();
     // ---- the products with K' and V'
     const dl4 t00 = delta_ld4(sT + c * CP + 4 * g), t10 = delta_ld4(sT + (16 + c) * CP + 4 * g), t11 = delta_ld4(sT + (16 + c) * CP + 16 + 4 * g);
     const dl4 m00 = delta_ld4(sM + c * CP + 4 * g), m10 = delta_ld4(sM + (16 + c) * CP + 4 * g), m11 = delta_ld4(sM + (16 + c) * CP + 16 + 4 * g);
@@ -730,6 +774,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(float* __restrict__ ws
 template <int NW, int DTW>
 struct DeltaFrags {
     dl4 w[2][DTW], q[2][DTW], k[DTW][2], y[2], gain[DTW];
+    float o[NW == 1 ? 2 : 1][4];               // what the chunk alone gives of o, for the tile (or both) that this wave finishes
 };
 
 template <int NW, int DTW>
@@ -774,20 +819,35 @@ __global__ __launch_bounds__(NW * kWave) void delta_scan_kernel(float* __restric
         }
 #pragma unroll
         for (int it = 0; it < 2; ++it) f.y[it] = t[(size_t)(6 * DTP + it * VTN + vt) * 64 + lane];
-    };
-    DeltaFrags<NW, DTW> now, next;
-    fetch(now, 0);
-    for (int ch = 0; ch < chunks; ++ch) {
-        if (ch + 1 < chunks) fetch(next, ch + 1);
-        // what the chunk alone gives of o, for the tile this wave finishes
-        float o0[NW == 1 ? 2 : 1][4];
 #pragma unroll
         for (int x = 0; x < (NW == 1 ? 2 : 1); ++x)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                const int i = 16 * (NW == 1 ? x : wave) + 4 * g + r;
-                o0[x][r] = (x < o_tiles && C * ch + i < count && col < V) ? o[((size_t)(first + C * ch + i) * H + head) * V + col] : 0.f;
+                // (what lies outside is read from the nearest place inside and never stored)
+                const int i = min(C * ch + 16 * (NW == 1 ? x : min(wave, 1)) + 4 * g + r, count - 1);
+                f.o[x][r] = o[((size_t)(first + i) * H + head) * V + min(col, V - 1)];
             }
+    };
+    // A chunk's o is stored while a later one is worked on, in front of what is asked for then: whoever waits for those loads
+    // (they are counted in order) waits for no store that has just begun.
+    float done[NW == 1 ? 2 : 1][4];
+    auto put = [&](int ch) {
+        if (o_tiles == 0 || col >= V) return;
+#pragma unroll
+        for (int x = 0; x < (NW == 1 ? 2 : 1); ++x) {
+            const int i = C * ch + 16 * (NW == 1 ? x : wave) + 4 * g;
+            float* p = o + ((size_t)(first + i) * H + head) * V + col;
+            if (C * ch + C <= count) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) p[(size_t)r * H * V] = done[x][r];
+            } else {
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    if (i + r < count) p[(size_t)r * H * V] = done[x][r];
+            }
+        }
+    };
+    auto work = [&](const DeltaFrags<NW, DTW>& f, int ch) {
         dl4 u[2], q[2];
 #pragma unroll
         for (int it = 0; it < 2; ++it) u[it] = q[it] = dl4{0.f, 0.f, 0.f, 0.f};
@@ -797,10 +857,10 @@ __global__ __launch_bounds__(NW * kWave) void delta_scan_kernel(float* __restric
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const float b = s[dt][e];
-                u[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.w[0][dt][e], b, u[0], 0, 0, 0);
-                u[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.w[1][dt][e], b, u[1], 0, 0, 0);
-                q[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.q[0][dt][e], b, q[0], 0, 0, 0);
-                q[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.q[1][dt][e], b, q[1], 0, 0, 0);
+                u[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.w[0][dt][e], b, u[0], 0, 0, 0);
+                u[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.w[1][dt][e], b, u[1], 0, 0, 0);
+                q[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.q[0][dt][e], b, q[0], 0, 0, 0);
+                q[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.q[1][dt][e], b, q[1], 0, 0, 0);
             }
         }
         if (NW > 1) {
@@ -809,7 +869,7 @@ __global__ __launch_bounds__(NW * kWave) void delta_scan_kernel(float* __restric
             buf[wave][1][lane] = u[1];
             buf[wave][2][lane] = q[0];
             buf[wave][3][lane] = q[1];
-            __syncthreads();
+            delta_lds_barrier();
 #pragma unroll
             for (int it = 0; it < 2; ++it) {
                 u[it] = buf[0][it][lane];
@@ -823,25 +883,43 @@ __global__ __launch_bounds__(NW * kWave) void delta_scan_kernel(float* __restric
             }
         }
 #pragma unroll
-        for (int it = 0; it < 2; ++it) u[it] += now.y[it];
+        for (int it = 0; it < 2; ++it) u[it] += f.y[it];
 #pragma unroll
         for (int x = 0; x < (NW == 1 ? 2 : 1); ++x)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int i = 16 * (NW == 1 ? x : wave) + 4 * g + r;
-                if (x < o_tiles && C * ch + i < count && col < V) o[((size_t)(first + C * ch + i) * H + head) * V + col] = o0[x][r] + q[x][r];
-            }
+            for (int r = 0; r < 4; ++r) done[x][r] = f.o[x][r] + q[x][r];
 #pragma unroll
-        for (int dt = 0; dt < DTW; ++dt) s[dt] *= now.gain[dt];
+        for (int dt = 0; dt < DTW; ++dt) s[dt] *= f.gain[dt];
 #pragma unroll
         for (int jt = 0; jt < 2; ++jt)
 #pragma unroll
             for (int e = 0; e < 4; ++e)
 #pragma unroll
                 for (int dt = 0; dt < DTW; ++dt)
-                    s[dt] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.k[dt][jt][e], u[jt][e], s[dt], 0, 0, 0);
-        now = next;
+                    s[dt] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.k[dt][jt][e], u[jt][e], s[dt], 0, 0, 0);
+    };
+    // AHEAD sets of fragments in turn: a chunk's are asked for AHEAD - 1 chunks before they are worked on
+    constexpr int AHEAD = DTW <= 2 ? 3 : 2;
+    DeltaFrags<NW, DTW> set[AHEAD];
+#pragma unroll
+    for (int k = 0; k < AHEAD; ++k) fetch(set[k], min(k, chunks - 1));
+    int ch0 = 0;
+    for (; ch0 + AHEAD <= chunks; ch0 += AHEAD) {          // (no branch around the loads: how many are newer is known where one is waited for)
+#pragma unroll
+        for (int k = 0; k < AHEAD; ++k) {
+            __builtin_amdgcn_sched_barrier(0);
+            work(set[k], ch0 + k);
+            put(ch0 + k);
+            fetch(set[k], min(ch0 + k + AHEAD, chunks - 1));
+            __builtin_amdgcn_sched_barrier(0);              // (the loads stay where they are)
+        }
     }
+#pragma unroll
+    for (int k = 0; k < AHEAD - 1; ++k)
+        if (ch0 + k < chunks) {
+            work(set[k], ch0 + k);
+            put(ch0 + k);
+        }
 #pragma unroll
     for (int dt = 0; dt < DTW; ++dt)
 #pragma unroll
