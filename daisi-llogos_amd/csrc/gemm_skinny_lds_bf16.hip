@@ -51,6 +51,8 @@ struct ActSource {
     int n_sums;
     int width;
     float eps;
+    int bounded;               // gated products: 0 silu(gate) * up; 1 both bounded by `limit` (see gated_value)
+    float limit;
 };
 
 // eight consecutive activations (k .. k + 7 of row m) as bf16
@@ -100,6 +102,16 @@ __device__ __forceinline__ uint4 produce8(const ActSource& src, int m, int k, in
 }
 
 typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
+
+// A gate and an up value as one: silu(gate) * up, or, bounded, with g = min(gate, limit) and u = up within -limit .. limit,
+// g * sigmoid(1.702 g) * (u + 1); with the hardware's exp2 and reciprocal.
+__device__ __forceinline__ float gated_value(float gate, float up, int bounded, float limit) {
+    if (bounded) {
+        const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+        return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.702f * 1.4426950408889634f * g)) * (u + 1.0f);
+    }
+    return gate * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * gate)) * up;
+}
 
 template <int RB, int MB, int MODE, typename TO, int CHUNK, int WAVES = kLdsWaves, bool PACKED = false, bool GATED = false>
 __global__ __launch_bounds__(WAVES * kWave) void gemm_skinny_lds_kernel(
@@ -267,7 +279,7 @@ __global__ __launch_bounds__(WAVES * kWave) void gemm_skinny_lds_kernel(
             for (int i = 0; i < 4; ++i) {
                 const float row_scale = MODE == PRODUCE_UNSCALED ? inv_rms[m] : 1.0f;
                 const float gate = acc[0][mb][i] * row_scale, up = xch[(((wave >> 1) * MB + mb) * 4 + i) * kWave + lane] * row_scale;
-                const float y = gate * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * gate)) * up;
+                const float y = gated_value(gate, up, src.bounded, src.limit);
                 if (col0 + i < N / 2) store_f32(out + (size_t)m * ldo + col0 + i, y);
             }
         }
@@ -441,16 +453,18 @@ LLOGOS_EXPORT int llogos_gemm_packed_bf16(void* out, int out_dtype, const void* 
 }
 
 // The same on a matrix packed with gate_rows (strips of gate and up rows in turn): out [M][ldo]
-// (ldo >= N / 2) = silu(a . gate^T) * (a . up^T) in bfloat16 or float32; plain activations, one
-// part, no bias.
+// (ldo >= N / 2) = silu(a . gate^T) * (a . up^T) in bfloat16 or float32, or with `bounded` the form of gated_value;
+// plain activations, one part, no bias.
 LLOGOS_EXPORT int llogos_gemm_packed_gated_bf16(void* out, int out_dtype, const void* act, int lda, const void* packed_w,
-                                                int M, int N, int K, int ldo, int chunk, hipStream_t stream) {
-    if (M <= 0 || N <= 0 || K <= 0 || (N % 32) || ldo < N / 2) return LLOGOS_BAD_ARGUMENT;
+                                                int M, int N, int K, int ldo, int chunk, int bounded, float limit, hipStream_t stream) {
+    if (M <= 0 || N <= 0 || K <= 0 || (N % 32) || (bounded && !(limit >= 0.f)) || ldo < N / 2) return LLOGOS_BAD_ARGUMENT;
     if (out_dtype != DT_BF16 && out_dtype != DT_F32) return LLOGOS_BAD_ARGUMENT;
     if (chunk != 128 && chunk != 256) return LLOGOS_BAD_ARGUMENT;
     if (M > 64 || (K % 8) || (lda % 8) || lda < K || ((uintptr_t)act % 16) || ((uintptr_t)packed_w % 16)) return LLOGOS_UNSUPPORTED;
     const int kpb = packed_k_per_block(K, 1, chunk);
     ActSource src{act, lda, 1, 0};
+    src.bounded = bounded;
+    src.limit = limit;
     const bf16_t* W = (const bf16_t*)packed_w;
     const int mb = (M + 15) / 16;
 #define GO(MB, CH) return launch_lds<1, MB, PRODUCE_PLAIN, CH, kLdsWaves, true, true>(out, out_dtype, src, W, nullptr, M, N, K, ldo, \
@@ -472,12 +486,12 @@ LLOGOS_EXPORT int llogos_gemm_packed_gated_bf16(void* out, int out_dtype, const 
 LLOGOS_EXPORT int llogos_gemm_packed_unscaled_bf16(void* out, int out_dtype, const void* act, int lda, const float* sums,
                                                    int n_sums, int width, float eps, const void* packed_w,
                                                    const float* bias, int M, int N, int K, int ldo,
-                                                   long long part_stride, int splits, int chunk, int gated,
-                                                   hipStream_t stream) {
+                                                   long long part_stride, int splits, int chunk, int gated, int bounded,
+                                                   float limit, hipStream_t stream) {
     if (M <= 0 || N <= 0 || K <= 0 || splits < 1 || n_sums < 1 || width < 1 || act == nullptr || sums == nullptr)
         return LLOGOS_BAD_ARGUMENT;
     if (out_dtype != DT_BF16 && out_dtype != DT_F32) return LLOGOS_BAD_ARGUMENT;
-    if (chunk != 128 && chunk != 256) return LLOGOS_BAD_ARGUMENT;
+    if ((chunk != 128 && chunk != 256) || (bounded && (!gated || !(limit >= 0.f)))) return LLOGOS_BAD_ARGUMENT;
     if (gated ? ((N % 32) || ldo < N / 2 || bias != nullptr) : ldo < N) return LLOGOS_BAD_ARGUMENT;
     if (M > kNormRows || (K % 8) || (lda % 8) || lda < K || ((uintptr_t)act % 16) || ((uintptr_t)packed_w % 16))
         return LLOGOS_UNSUPPORTED;
@@ -486,6 +500,8 @@ LLOGOS_EXPORT int llogos_gemm_packed_unscaled_bf16(void* out, int out_dtype, con
         return LLOGOS_BAD_ARGUMENT;
     const int kpb = packed_k_per_block(K, parts, chunk);
     ActSource src{act, lda, 1, 0, sums, n_sums, width, eps};
+    src.bounded = bounded;
+    src.limit = limit;
     const bf16_t* W = (const bf16_t*)packed_w;
 #define GO(CH, GATED) return launch_lds<1, 1, PRODUCE_UNSCALED, CH, kLdsWaves, true, GATED>(out, out_dtype, src, W, bias, M, N, K, ldo, \
                                                                                             (size_t)part_stride, kpb, parts, stream)

@@ -63,6 +63,14 @@ __device__ __forceinline__ uint32_t tiles_pack_bf16(float lo, float hi) {
     const f32x2_t v = {lo, hi};
     return __builtin_bit_cast(uint32_t, __builtin_convertvector(v, bf16x2_t));
 }
+// silu(gate) * up, or, with limit >= 0, g = min(gate, limit), u = up within -limit .. limit, g * sigmoid(1.702 g) * (u + 1)
+__device__ __forceinline__ float tiles_gated(float gate, float up, float limit) {
+    if (limit >= 0.f) {
+        const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+        return g / (1.0f + __expf(-1.702f * g)) * (u + 1.0f);
+    }
+    return gate / (1.0f + __expf(-gate)) * up;
+}
 #define SB() __builtin_amdgcn_sched_barrier(0)
 
 template <int N> __device__ __forceinline__ void tiles_wait_loads() {
@@ -77,7 +85,7 @@ template <int TM, typename TO, int EPI>
 __device__ __forceinline__ void tile_body(
         unsigned char* tiles_lds, TO* __restrict__ out, const bf16_t* __restrict__ a, int lda,
         const unsigned char* __restrict__ wp, const float* __restrict__ bias, int M, int N, int K, int ldo,
-        int n_row_blocks, int m_tile, int n_tile, int stage_begin, int stage_end) {
+        int n_row_blocks, int m_tile, int n_tile, int stage_begin, int stage_end, float limit) {
     constexpr int BM = kWavesM * TM * 32;
     constexpr int kStageBytes = kStageW + BM * kStageK * 2;
     constexpr int kPieces = 4 + TM;                                          // copies per wave and stage: 4 of w, TM of the activations
@@ -238,7 +246,7 @@ __device__ __forceinline__ void tile_body(
 #pragma unroll
                     for (int e = 0; e < 4; ++e) {
                         const float gt = acc[tt][rt][4 * q + e], u = acc[tt][rt][8 + 4 * q + e];
-                        y[e] = gt / (1.0f + __expf(-gt)) * u;
+                        y[e] = tiles_gated(gt, u, limit);
                     }
                     if (sizeof(TO) == 2 && col + 3 < N / 2 && ((ldo & 3) == 0) && ((reinterpret_cast<uintptr_t>(out) & 7) == 0)) {
                         uint2 pk;
@@ -287,7 +295,7 @@ template <typename TO, int EPI>
 __global__ __launch_bounds__(kTileWaves * kWave) void gemm_tiles_kernel(
         TO* __restrict__ out, const bf16_t* __restrict__ a, int lda, const unsigned char* __restrict__ wp,
         const float* __restrict__ bias, int M, int N, int K, int ldo, size_t part_stride, int n_row_blocks,
-        int m_tiles4, int m_tiles2, int n_full, int n_tiles, int blocks4, int parts) {
+        int m_tiles4, int m_tiles2, int n_full, int n_tiles, int blocks4, int parts, float limit) {
     extern __shared__ __attribute__((aligned(1024))) unsigned char tiles_lds[];
     const int stages = K / kStageK;
     const bool big = (int)blockIdx.x < blocks4;
@@ -301,8 +309,8 @@ __global__ __launch_bounds__(kTileWaves * kWave) void gemm_tiles_kernel(
     // when there are at least as many stages as parts
     const int s0 = (int)((long long)stages * part / parts), s1 = (int)((long long)stages * (part + 1) / parts);
     TO* dst = out + (size_t)part * part_stride;
-    if (big) tile_body<4, TO, EPI>(tiles_lds, dst, a, lda, wp, bias, M, N, K, ldo, n_row_blocks, m_tile, n_tile, s0, s1);
-    else tile_body<2, TO, EPI>(tiles_lds, dst, a, lda, wp, bias, M, N, K, ldo, n_row_blocks, m_tile, n_tile, s0, s1);
+    if (big) tile_body<4, TO, EPI>(tiles_lds, dst, a, lda, wp, bias, M, N, K, ldo, n_row_blocks, m_tile, n_tile, s0, s1, limit);
+    else tile_body<2, TO, EPI>(tiles_lds, dst, a, lda, wp, bias, M, N, K, ldo, n_row_blocks, m_tile, n_tile, s0, s1, limit);
 }
 
 // How the tiles are cut: row tiles 0 .. n_full - 1 in tiles of 256 tokens, the rest in tiles of 128 tokens.
@@ -319,7 +327,7 @@ static int tiles_n_full(int n_tiles, int m_tiles4, int parts, int token_tiles, i
 
 template <typename TO, int EPI>
 static int launch_tiles(void* out, const void* a, int lda, const void* wp, const float* bias, int M, int N, int K,
-                        int ldo, long long part_stride, int parts, int token_tiles, int compute_units, hipStream_t stream) {
+                        int ldo, long long part_stride, int parts, int token_tiles, int compute_units, float limit, hipStream_t stream) {
     const int n_row_blocks = (N + 63) / 64, n_tiles = (n_row_blocks + kWavesN - 1) / kWavesN;
     const int m4 = (M + 255) / 256, m2 = (M + 127) / 128;
     const int n_full = tiles_n_full(n_tiles, m4, parts, token_tiles, compute_units);
@@ -336,18 +344,18 @@ static int launch_tiles(void* out, const void* a, int lda, const void* wp, const
     }
     gemm_tiles_kernel<TO, EPI><<<blocks4 + blocks2, kTileWaves * kWave, smem, stream>>>(
         (TO*)out, (const bf16_t*)a, lda, (const unsigned char*)wp, bias, M, N, K, ldo, (size_t)part_stride, n_row_blocks,
-        m4, m2, n_full, n_tiles, blocks4, parts);
+        m4, m2, n_full, n_tiles, blocks4, parts, limit);
     return LLOGOS_LAUNCH_CHECK();
 }
 
 // a: bfloat16 [M][lda]; packed_w: llogos_pack_weights of w [N][K]; out [parts][M][ldo] bfloat16 or float32.
 // epilogue 0: out = a . w^T (+ bias [N]); 1: w's 16-row strips alternate gate and up rows, out is
-// [M][N / 2] = silu(gate) * up (no bias, one part).  parts > 1: float32 partial sums over ranges of k, part_stride
+// [M][N / 2] = silu(gate) * up, or with limit >= 0 the form of tiles_gated (no bias, one part).  parts > 1: float32 partial sums over ranges of k, part_stride
 // elements apart, no bias.  token_tiles: see tiles_n_full.  compute_units: of the GPU, for that choice.
 // K must be a multiple of 64 and every part must hold at least two stages of 64.
 LLOGOS_EXPORT int llogos_gemm_tiles_bf16(void* out, int out_dtype, const void* a, int lda, const void* packed_w,
                                          const float* bias, int M, int N, int K, int ldo, long long part_stride,
-                                         int epilogue, int parts, int token_tiles, int compute_units, hipStream_t stream) {
+                                         int epilogue, int parts, int token_tiles, int compute_units, float limit, hipStream_t stream) {
     if (M <= 0 || N <= 0 || K <= 0 || out == nullptr || a == nullptr || packed_w == nullptr) return LLOGOS_BAD_ARGUMENT;
     if (out_dtype != DT_BF16 && out_dtype != DT_F32) return LLOGOS_BAD_ARGUMENT;
     if (epilogue != EPI_PLAIN && epilogue != EPI_SWIGLU) return LLOGOS_BAD_ARGUMENT;
@@ -358,8 +366,8 @@ LLOGOS_EXPORT int llogos_gemm_tiles_bf16(void* out, int out_dtype, const void* a
     if (parts < 1 || compute_units < 1) return LLOGOS_BAD_ARGUMENT;
     if (parts > 1 && (out_dtype != DT_F32 || bias != nullptr || part_stride < (long long)M * ldo)) return LLOGOS_BAD_ARGUMENT;
     if (parts > 1 && (K / kStageK) / parts < 2) return LLOGOS_UNSUPPORTED;          // every part holds two stages or more
-#define GO(EPI) do { if (out_dtype == DT_BF16) return launch_tiles<bf16_t, EPI>(out, a, lda, packed_w, bias, M, N, K, ldo, part_stride, parts, token_tiles, compute_units, stream); \
-                     return launch_tiles<float, EPI>(out, a, lda, packed_w, bias, M, N, K, ldo, part_stride, parts, token_tiles, compute_units, stream); } while (0)
+#define GO(EPI) do { if (out_dtype == DT_BF16) return launch_tiles<bf16_t, EPI>(out, a, lda, packed_w, bias, M, N, K, ldo, part_stride, parts, token_tiles, compute_units, limit, stream); \
+                     return launch_tiles<float, EPI>(out, a, lda, packed_w, bias, M, N, K, ldo, part_stride, parts, token_tiles, compute_units, limit, stream); } while (0)
     if (epilogue == EPI_SWIGLU) GO(EPI_SWIGLU);
     GO(EPI_PLAIN);
 #undef GO

@@ -5,10 +5,10 @@
 // sum v itself is left in `delta`, float [T, H].  A factor on the sum belongs into wa and wb.  All arithmetic is 32-bit.
 #include "common.h"
 
-constexpr int kPairParts = 8;          // parts of a product whose loads are in flight together
+constexpr int kPairParts = 8;          // parts of a product whose loads are in flight together, where either comes in parts
 
-// One block a row; a thread keeps its ITEMS values of the row in registers from pass to pass.
-template <typename TA, typename TB, typename TH, int ITEMS>
+// One block a row; a thread keeps its ITEMS values of the row in registers from pass to pass.  PARTS: 1 or kPairParts.
+template <typename TA, typename TB, typename TH, int ITEMS, int PARTS>
 __global__ __launch_bounds__(1024) void pair_norm_kernel(float* __restrict__ x, const TA* __restrict__ a, int a_parts, size_t a_stride,
                                                          const TB* __restrict__ b, int b_parts, size_t b_stride,
                                                          const float* __restrict__ wa, const float* __restrict__ wb, float eps,
@@ -17,7 +17,7 @@ __global__ __launch_bounds__(1024) void pair_norm_kernel(float* __restrict__ x, 
     __shared__ float red[16];
     const size_t r = blockIdx.x;
     float va[ITEMS], vb[ITEMS], xv[ITEMS], fa[ITEMS], fb[ITEMS], fn[ITEMS];
-    float pa[ITEMS][kPairParts], pb[ITEMS][kPairParts];
+    float pa[ITEMS][PARTS], pb[ITEMS][PARTS];
 #pragma unroll
     for (int it = 0; it < ITEMS; ++it) {
         const int i = it * blockDim.x + threadIdx.x;
@@ -27,7 +27,7 @@ __global__ __launch_bounds__(1024) void pair_norm_kernel(float* __restrict__ x, 
         fb[it] = ok ? wb[i] : 0.f;
         fn[it] = (ok && wn) ? wn[i] : 0.f;
 #pragma unroll
-        for (int q = 0; q < kPairParts; ++q) {
+        for (int q = 0; q < PARTS; ++q) {
             pa[it][q] = (ok && q < a_parts) ? load_f32(a + q * a_stride + r * H + i) : 0.f;
             pb[it][q] = (ok && q < b_parts) ? load_f32(b + q * b_stride + r * H + i) : 0.f;
         }
@@ -38,10 +38,10 @@ __global__ __launch_bounds__(1024) void pair_norm_kernel(float* __restrict__ x, 
         const int i = it * blockDim.x + threadIdx.x;
         float ta = pa[it][0], tb = pb[it][0];
 #pragma unroll
-        for (int q = 1; q < kPairParts; ++q) { ta += pa[it][q]; tb += pb[it][q]; }       // ascending order
+        for (int q = 1; q < PARTS; ++q) { ta += pa[it][q]; tb += pb[it][q]; }       // ascending order
         if (i < H) {
-            for (int q = kPairParts; q < a_parts; ++q) ta += load_f32(a + q * a_stride + r * H + i);
-            for (int q = kPairParts; q < b_parts; ++q) tb += load_f32(b + q * b_stride + r * H + i);
+            for (int q = PARTS; q < a_parts; ++q) ta += load_f32(a + q * a_stride + r * H + i);
+            for (int q = PARTS; q < b_parts; ++q) tb += load_f32(b + q * b_stride + r * H + i);
         }
         va[it] = ta;
         vb[it] = tb;
@@ -78,8 +78,9 @@ LLOGOS_EXPORT int llogos_pair_norm(float* x, const void* a, int a_dtype, int a_p
     int items = T >= 256 ? 4 : 1;
     while ((H + items - 1) / items > 1024) items *= 2;
     const int threads = ((H + items - 1) / items + kWave - 1) / kWave * kWave;
-#define PN(TA, TB, TH, IT) pair_norm_kernel<TA, TB, TH, IT><<<T, threads, 0, stream>>>(x, (const TA*)a, a_parts, (size_t)a_stride, \
+#define PNP(TA, TB, TH, IT, PARTS) pair_norm_kernel<TA, TB, TH, IT, PARTS><<<T, threads, 0, stream>>>(x, (const TA*)a, a_parts, (size_t)a_stride, \
         (const TB*)b, b_parts, (size_t)b_stride, wa, wb, eps, wn, eps_n, (TH*)h, delta, H)
+#define PN(TA, TB, TH, IT) do { if (a_parts == 1 && b_parts == 1) PNP(TA, TB, TH, IT, 1); else PNP(TA, TB, TH, IT, kPairParts); } while (0)
 #define PNI(TA, TB, TH) do { if (items == 1) PN(TA, TB, TH, 1); else if (items == 2) PN(TA, TB, TH, 2); else if (items == 4) PN(TA, TB, TH, 4); \
         else if (items == 8) PN(TA, TB, TH, 8); else PN(TA, TB, TH, 16); } while (0)
     if (h && h_dtype != DT_F32 && h_dtype != DT_BF16) return LLOGOS_BAD_ARGUMENT;
@@ -91,5 +92,6 @@ LLOGOS_EXPORT int llogos_pair_norm(float* x, const void* a, int a_dtype, int a_p
     else return LLOGOS_BAD_ARGUMENT;
 #undef PNI
 #undef PN
+#undef PNP
     return LLOGOS_LAUNCH_CHECK();
 }

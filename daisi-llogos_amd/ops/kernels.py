@@ -1705,9 +1705,11 @@ def pack_weights(w: torch.Tensor, gate_rows: int = 0) -> PackedWeight:
     return PackedWeight(data, N, K, int(gate_rows))
 
 
-def gemm_packed_gated_bf16(a: torch.Tensor, pw: PackedWeight, out_dtype: torch.dtype, chunk: int = 256) -> Optional[torch.Tensor]:
+def gemm_packed_gated_bf16(a: torch.Tensor, pw: PackedWeight, out_dtype: torch.dtype, chunk: int = 256,
+                           limit: Optional[float] = None) -> Optional[torch.Tensor]:
     """silu(a . gate^T) * (a . up^T) as [M, gate_rows] for up to 64 rows of bfloat16 activations, on a matrix
-    packed with gate_rows: the gate/up product stays in registers.  None for shapes it does not take."""
+    packed with gate_rows: the gate/up product stays in registers.  With `limit` the form of clamped_glu instead.
+    None for shapes it does not take."""
     if pw.gate_rows <= 0 or a.dtype != torch.bfloat16 or a.dim() != 2:
         return None
     M, K = a.shape
@@ -1718,7 +1720,7 @@ def gemm_packed_gated_bf16(a: torch.Tensor, pw: PackedWeight, out_dtype: torch.d
     _need(a.is_cuda and a.device == pw.data.device, "gemm: a and w must be on the same GPU")
     out = torch.empty((M, pw.gate_rows), dtype=out_dtype, device=a.device)
     code = _lib().llogos_gemm_packed_gated_bf16(_p(out), _DT[out_dtype], _p(a), a.stride(0), _p(pw.data), M, pw.N, K,
-                                                pw.gate_rows, int(chunk), _stream())
+                                                pw.gate_rows, int(chunk), int(limit is not None), ctypes.c_float(limit or 0.0), _stream())
     if code == -2:
         return None
     _check(code, "gemm_packed_gated_bf16")
@@ -1857,11 +1859,12 @@ def gemm_residual_bf16(x: torch.Tensor, a: torch.Tensor, pw: PackedWeight, bias:
 
 
 def gemm_packed_unscaled_bf16(squares: RowSquares, eps: float, pw: PackedWeight, bias: Optional[torch.Tensor],
-                              out_dtype: torch.dtype, splits: int = 1, chunk: int = 128) -> Optional[torch.Tensor]:
+                              out_dtype: torch.dtype, splits: int = 1, chunk: int = 128,
+                              limit: Optional[float] = None) -> Optional[torch.Tensor]:
     """The few-row product on packed weights with an rmsnorm's rows as its activations, of which `squares`
     holds x * norm_w in bfloat16 and the sums of squares of x (gemm_residual_bf16 with norm_w): the rows'
     scale 1 / sqrt(mean square + eps) is applied to the product, in float32.  On a matrix packed with
-    gate_rows the result is silu(gate) * up [M, gate_rows], otherwise [parts, M, N] as gemm_packed_bf16 (a
+    gate_rows the result is silu(gate) * up [M, gate_rows] (with `limit` the form of clamped_glu), otherwise [parts, M, N] as gemm_packed_bf16 (a
     bias is added after the scale).  None for shapes it does not take."""
     a = squares.unscaled
     if a is None:
@@ -1895,7 +1898,7 @@ def gemm_packed_unscaled_bf16(squares: RowSquares, eps: float, pw: PackedWeight,
     code = lib.llogos_gemm_packed_unscaled_bf16(
         _p(out), _DT[out_dtype], _p(a), a.stride(0), _p(squares.sums), squares.sums.shape[0], K,
         ctypes.c_float(eps), _p(pw.data), _p(bias), M, N, K, cols, ctypes.c_longlong(M * N), int(splits), int(chunk),
-        int(gated), _stream())
+        int(gated), int(gated and limit is not None), ctypes.c_float(limit or 0.0), _stream())
     if code == -2:
         return None
     _check(code, "gemm_packed_unscaled_bf16")
@@ -1944,10 +1947,10 @@ def tiles_plan(M: int, N: int, K: int) -> Optional[Tuple[int, int]]:
 
 
 def gemm_tiles_bf16(a: torch.Tensor, pw: PackedWeight, bias: Optional[torch.Tensor], out_dtype: torch.dtype,
-                    parts: int = 1, token_tiles: int = 0) -> Optional[torch.Tensor]:
+                    parts: int = 1, token_tiles: int = 0, limit: Optional[float] = None) -> Optional[torch.Tensor]:
     """a [M, K] . w^T on the packed copy of w for any number of rows (tiles of 256 or 128 tokens x 256 rows,
     v_mfma_f32_32x32x16_bf16): [M, N] with the bias added, or, for a matrix packed with gate_rows,
-    [M, gate_rows] = silu(gate) * up; with parts > 1 float32 partial sums [parts, M, N] over ranges of k.
+    [M, gate_rows] = silu(gate) * up (with `limit` the form of clamped_glu); with parts > 1 float32 partial sums [parts, M, N] over ranges of k.
     token_tiles: 4 or 2 force tiles of 256 or 128 tokens, 0 lets the launch choose.
     None for shapes it does not take (K no multiple of 64, parts of fewer than 128 values of k)."""
     if a.dtype != torch.bfloat16 or a.dim() != 2:
@@ -1969,7 +1972,7 @@ def gemm_tiles_bf16(a: torch.Tensor, pw: PackedWeight, bias: Optional[torch.Tens
     out = torch.empty((parts, M, width), dtype=out_dtype, device=a.device)
     code = _lib().llogos_gemm_tiles_bf16(_p(out), _DT[out_dtype], _p(a), a.stride(0), _p(pw.data), _p(bias), M, pw.N, K,
                                          width, ctypes.c_longlong(M * width), int(gated), int(parts), int(token_tiles),
-                                         compute_units(a.device), _stream())
+                                         compute_units(a.device), ctypes.c_float(-1.0 if limit is None else limit), _stream())
     if code == -2:
         return None
     _check(code, "gemm_tiles_bf16")

@@ -138,8 +138,8 @@ class Linear(Part):
         norm_w = residual.norm.row_weight() if residual.norm is not None else None
         return K.gemm_residual_bf16(x, a, self.packed, self.bias, waves, norm_w, strips)
 
-    def gated_product(self, a) -> Optional[torch.Tensor]:
-        """silu(a . gate^T) * (a . up^T) as [M, out] in the runtime's type, made in one kernel from the
+    def gated_product(self, a, limit: Optional[float] = None) -> Optional[torch.Tensor]:
+        """silu(a . gate^T) * (a . up^T), or with `limit` the bounded form of ops.kernels.clamped_glu, as [M, out] in the runtime's type, made in one kernel from the
         packed copy (up to 64 rows the weight-streaming product, for prompts the tiled one); None where that
         does not apply (no packed copy, float32, row counts at which the library's product and a SwiGLU pass
         are faster)."""
@@ -147,12 +147,12 @@ class Linear(Part):
             return None
         if isinstance(a, NormedRows):
             return K.gemm_packed_unscaled_bf16(a.squares, a.eps, self.packed, None, self.rt.dtype, 1,
-                                               K.packed_plan(a.x.shape[0], self.packed.N, self.packed.K)[1])
+                                               K.packed_plan(a.x.shape[0], self.packed.N, self.packed.K)[1], limit=limit)
         if a.dim() != 2:
             return None
         if a.shape[0] > K.SKINNY_MAX_ROWS:
-            return K.gemm_tiles_bf16(a, self.packed, None, self.rt.dtype) if K.tiles_serve_gated(a.shape[0], a.shape[1]) else None
-        return K.gemm_packed_gated_bf16(a, self.packed, self.rt.dtype, K.packed_plan(a.shape[0], self.packed.N, self.packed.K)[1])
+            return K.gemm_tiles_bf16(a, self.packed, None, self.rt.dtype, limit=limit) if K.tiles_serve_gated(a.shape[0], a.shape[1]) else None
+        return K.gemm_packed_gated_bf16(a, self.packed, self.rt.dtype, K.packed_plan(a.shape[0], self.packed.N, self.packed.K)[1], limit=limit)
 
     def bias_rows(self, rows_out: Optional[int] = None) -> Optional[torch.Tensor]:
         return self.bias if (self.bias is None or rows_out is None) else self.bias[:rows_out]

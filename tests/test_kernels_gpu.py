@@ -842,7 +842,7 @@ def test_tiled_product_cuts_the_last_round_into_smaller_tiles():
     for units in (64, 256, 1):                    # 224 tiles: 3.5 rounds of 64 (cut), less than one round of 256, whole rounds of 1
         out = torch.empty((M, N), dtype=torch.float32, device=a.device)
         code = lib.llogos_gemm_tiles_bf16(K._p(out), K.F32, K._p(a), a.stride(0), K._p(pw.data), None, M, N, K_, N, M * N, 0, 1, 0,
-                                          units, K._stream())
+                                          units, -1.0, K._stream())
         assert code == 0
         outs.append(out)
     _close(outs[0], _np(a) @ _np(w).T, "float32", scale=np.abs(_np(a) @ _np(w).T).max() * 10)

@@ -309,8 +309,15 @@ def test_two_normed_outputs_join_the_stream(T, N, pa, pb, rows):
 
 
 @pytest.mark.parametrize("dtype", H.DTYPES)
-@pytest.mark.parametrize("hidden,ff,limit,T", [(48, 33, 0.5, 5), (96, 64, 1.5, 70), (64, 40, 1e9, 3), (128, 96, 0.0, 130)])
-def test_the_bounded_feed_forward_alone(hidden, ff, limit, T, dtype):
+@pytest.mark.parametrize("hidden,ff,limit,T", [(48, 33, 0.5, 5), (96, 64, 1.5, 70), (64, 40, 1e9, 3), (128, 96, 0.0, 130), (64, 64, 1.2, 40), (256, 160, 0.8, 16),
+                                                  (128, 96, 1.0, 1100), (64, 48, 0.0, 2)])
+@pytest.mark.parametrize("fused", [True, False])
+def test_the_bounded_feed_forward_alone(hidden, ff, limit, T, fused, dtype, monkeypatch):
+    """The bounds in the products' epilogues (few rows, prompts of the tiled product, rows without their norm's scale) and in
+    a kernel behind them."""
+    monkeypatch.setattr(P.ClampedGLU, "fuse_from", 0 if fused else 1 << 30)
+    if dtype == "bfloat16" and fused and ff % 16 == 0 and (T <= 64 or 1024 <= T <= 2048) and hidden % 64 == 0:
+        monkeypatch.setattr(K, "clamped_glu", lambda *a, _k=K.clamped_glu: _k(*a) if a[0].shape[-1] == 10 else pytest.fail("not fused"))
     rng = np.random.default_rng(ff)
     mlp = P.ClampedGLU(prefix="f.", hidden=hidden, intermediate=ff, limit=limit)
     plain = _bind(mlp, rng, dtype)
@@ -324,6 +331,18 @@ def test_the_bounded_feed_forward_alone(hidden, ff, limit, T, dtype):
     if 0.0 < limit < 10.0:                                     # both bounds are met, on the gate only from above
         for other in (limit * 1.1, limit * 0.9):
             assert np.abs(pz.clamped_ff(h, pz.part(plain, "f."), other) - want).max() > 30 * PART_TOL["float32"] * np.abs(want).max()
+    if dtype == "bfloat16" and T <= 16 and hidden % 8 == 0 and ff % 16 == 0:
+        # behind a product that has added itself to the stream: the norm's rows come without their scale
+        before = P.Linear(["w"], 64, [hidden], suffix="")
+        nxt = P.RMSNorm(name="n", width=hidden, eps=1e-3, suffix="")
+        w = {"w": torch.tensor(rng.standard_normal((hidden, 64)) * 0.3, dtype=torch.bfloat16), "n": torch.tensor(rng.uniform(0.5, 1.5, hidden), dtype=torch.bfloat16)}
+        before.bind(w.get, mlp.rt); nxt.bind(w.get, mlp.rt)
+        xt = _f32(rng.standard_normal((T, hidden)))
+        left = before.add_to(torch.tensor(rng.standard_normal((T, 64)), dtype=torch.bfloat16, device=DEV), base.Residual(xt, nxt))
+        rows = nxt.forward(xt, left, lazy=True)
+        assert isinstance(rows, base.NormedRows)
+        full = pz.clamped_ff(pz.norm(_np(xt), w["n"].double().numpy(), 1e-3), pz.part(plain, "f."), limit)
+        _close(_np(K.sum_parts(mlp.forward(None, rows), None, torch.float32)), full, PART_TOL[dtype])
     z = rng.standard_normal((3, 4, 10)) * 3.0
     g, u = np.minimum(z.sum(0)[:, :5], 1.25), np.clip(z.sum(0)[:, 5:], -1.25, 1.25)
     _close(_np(K.clamped_glu(_f32(z), 1.25, DT[dtype])), g * pz.sigmoid(1.702 * g) * (u + 1.0), PART_TOL[dtype])
