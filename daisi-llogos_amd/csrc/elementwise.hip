@@ -406,8 +406,8 @@ __global__ void qk_rope_cache_kernel(const TI* __restrict__ qkv, int parts, size
     }
 }
 
-// The same for head_dim = rot = 128 with split-half pairing, without LDS or block barriers, for
-// prompts.  With one (token, head) a wave and two values a lane this kernel took 29.5 us for 2,048
+// The same for head_dim = 128, rotated whole in split halves or (NEAR) the first `rot` dimensions, a
+// multiple of 4, in neighbouring pairs, without LDS or block barriers, for prompts.  With one (token, head) a wave and two values a lane this kernel took 29.5 us for 2,048
 // tokens of the 8B head shape (2.6 TB/s) and 20 us of that with every store left out: its time
 // was the number of its load instructions (five a token and head, of 4 and 8 bytes a lane), not
 // bytes or latency.  So a lane takes four consecutive dimensions (one 16-byte load), half a
@@ -436,13 +436,13 @@ template <> __device__ __forceinline__ void store4_f32<bf16_t>(bf16_t* p, float 
     *reinterpret_cast<uint2*>(p) = v;
 }
 
-template <typename TI, typename T>
+template <typename TI, typename T, bool NEAR>
 __global__ __launch_bounds__(kWave * kRopeHeadsPerBlock / 2) void qk_rope_cache_hd128_kernel(
         const TI* __restrict__ qkv, int parts, size_t part_stride, int row_stride,
         const float* __restrict__ bias, T* __restrict__ q_out, int n_heads, int n_kv_heads,
         const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w,
         float eps, const float2* __restrict__ cs, T* __restrict__ k_pool, T* __restrict__ v_pool, PagedKV cache,
-        const int* __restrict__ tok_seq, const int* __restrict__ tok_pos, int n_tokens) {
+        const int* __restrict__ tok_seq, const int* __restrict__ tok_pos, int n_tokens, int rot) {
     constexpr int HD = 128;
     const int t0 = blockIdx.x * kRopeTokens;
     const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
@@ -467,10 +467,13 @@ __global__ __launch_bounds__(kWave * kRopeHeadsPerBlock / 2) void qk_rope_cache_
             const float4 more = load4_f32<TI>(src + q * part_stride);
             x[i].x += more.x; x[i].y += more.y; x[i].z += more.z; x[i].w += more.w;
         }
-        // (cos, sin) of dimensions d & 63 .. + 3: two 16-byte loads
-        const float4* c4 = reinterpret_cast<const float4*>(cs + (size_t)t * 64 + (d & 63));
-        ca[i] = c4[0];
-        cb[i] = c4[1];
+        if (NEAR) {                                         // (cos, sin) of the lane's two pairs; the rest of a head passes
+            ca[i] = d < rot ? *reinterpret_cast<const float4*>(cs + (size_t)t * (rot / 2) + d / 2) : make_float4(1.f, 0.f, 1.f, 0.f);
+        } else {                                            // (cos, sin) of dimensions d & 63 .. + 3: two 16-byte loads
+            const float4* c4 = reinterpret_cast<const float4*>(cs + (size_t)t * 64 + (d & 63));
+            ca[i] = c4[0];
+            cb[i] = c4[1];
+        }
         seq[i] = tok_seq[t];
         pos[i] = tok_pos[t];
     }
@@ -528,11 +531,15 @@ __global__ __launch_bounds__(kWave * kRopeHeadsPerBlock / 2) void qk_rope_cache_
             const float inv = 1.0f / sqrtf(ss / (float)HD + eps);
             a.x = a.x * inv * w.x; a.y = a.y * inv * w.y; a.z = a.z * inv * w.z; a.w = a.w * inv * w.w;
         }
-        float4 p;
-        p.x = __shfl_xor(a.x, 16, kWave); p.y = __shfl_xor(a.y, 16, kWave);
-        p.z = __shfl_xor(a.z, 16, kWave); p.w = __shfl_xor(a.w, 16, kWave);
-        float4 y;
-        if (l < 16) {
+        float4 p, y;
+        if (!NEAR) {
+            p.x = __shfl_xor(a.x, 16, kWave); p.y = __shfl_xor(a.y, 16, kWave);
+            p.z = __shfl_xor(a.z, 16, kWave); p.w = __shfl_xor(a.w, 16, kWave);
+        }
+        if (NEAR) {
+            y.x = a.x * ca[i].x - a.y * ca[i].y; y.y = a.x * ca[i].y + a.y * ca[i].x;
+            y.z = a.z * ca[i].z - a.w * ca[i].w; y.w = a.z * ca[i].w + a.w * ca[i].z;
+        } else if (l < 16) {
             y.x = a.x * ca[i].x - p.x * ca[i].y; y.y = a.y * ca[i].z - p.y * ca[i].w;
             y.z = a.z * cb[i].x - p.z * cb[i].y; y.w = a.w * cb[i].z - p.w * cb[i].w;
         } else {
@@ -566,17 +573,20 @@ LLOGOS_EXPORT int llogos_qk_rope_cache(const void* qkv, int in_dtype, int parts,
     const int total_heads = n_heads + 2 * n_kv_heads;
     dim3 grid(T, (total_heads + kHeadsPerBlock - 1) / kHeadsPerBlock), block(kWave, kHeadsPerBlock);
     dim3 grid128((T + kRopeTokens - 1) / kRopeTokens, (total_heads + kRopeHeadsPerBlock - 1) / kRopeHeadsPerBlock);
-    // (the wide form takes 16-byte steps through rows, tables and pools)
-    const bool wide = head_dim == 128 && rot == 128 && pairing == 0 && (row_stride % 4) == 0 && (part_stride % 4) == 0 &&
+    // (the wide form takes 16-byte steps through rows, tables and pools; few tokens
+    // leave it too few blocks for its waits: 8 rows in parts 27 us against 14, another mixer's kernels beside it)
+    const bool wide = head_dim == 128 && (pairing == 0 ? rot == 128 : (T > 64 && rot > 0 && rot % 4 == 0)) &&
+                      (row_stride % 4) == 0 && (part_stride % 4) == 0 &&
                       ((uintptr_t)qkv % 16) == 0 && ((uintptr_t)q_out % 16) == 0 && ((uintptr_t)cs % 16) == 0 &&
                       ((uintptr_t)bias % 16) == 0 && ((uintptr_t)k_pool % 16) == 0 && ((uintptr_t)v_pool % 16) == 0 &&
                       ((uintptr_t)q_norm_w % 16) == 0 && ((uintptr_t)k_norm_w % 16) == 0;
     const size_t smem = (size_t)kHeadsPerBlock * head_dim * sizeof(float);
-#define LAUNCH(TI, T_) do { \
-        if (wide) \
-            qk_rope_cache_hd128_kernel<TI, T_><<<grid128, kWave * kRopeHeadsPerBlock / 2, 0, stream>>>( \
+#define LAUNCH_WIDE(TI, T_, NEAR) qk_rope_cache_hd128_kernel<TI, T_, NEAR><<<grid128, kWave * kRopeHeadsPerBlock / 2, 0, stream>>>( \
                 (const TI*)qkv, parts, (size_t)part_stride, row_stride, bias, (T_*)q_out, n_heads, n_kv_heads, \
-                q_norm_w, k_norm_w, eps, (const float2*)cs, (T_*)k_pool, (T_*)v_pool, cache, tok_seq, tok_pos, T); \
+                q_norm_w, k_norm_w, eps, (const float2*)cs, (T_*)k_pool, (T_*)v_pool, cache, tok_seq, tok_pos, T, rot)
+#define LAUNCH(TI, T_) do { \
+        if (wide && pairing == 0) LAUNCH_WIDE(TI, T_, false); \
+        else if (wide) LAUNCH_WIDE(TI, T_, true); \
         else \
             qk_rope_cache_kernel<TI, T_><<<grid, block, smem, stream>>>( \
                 (const TI*)qkv, parts, (size_t)part_stride, row_stride, bias, (T_*)q_out, n_heads, n_kv_heads, head_dim, \
@@ -587,6 +597,7 @@ LLOGOS_EXPORT int llogos_qk_rope_cache(const void* qkv, int in_dtype, int parts,
     else if (dtype == DT_BF16 && in_dtype == DT_F32) LAUNCH(float, bf16_t);
     else return LLOGOS_BAD_ARGUMENT;
 #undef LAUNCH
+#undef LAUNCH_WIDE
     return LLOGOS_LAUNCH_CHECK();
 }
 

@@ -2055,7 +2055,7 @@ def gemm_product(a: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, swigl
         if f32_ok:
             return torch.mm(a, w.t(), out_dtype=torch.float32)
         return torch.matmul(a, w.t())
-    return gemm_generic(a, w, None, out_dtype)
+    return gemm_generic(a, w, None, torch.float32 if f32_ok else out_dtype)
 
 
 def gemm_library_add(x: torch.Tensor, a: torch.Tensor, w: torch.Tensor, packed: Optional[PackedWeight] = None) -> bool:

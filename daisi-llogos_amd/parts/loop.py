@@ -41,6 +41,8 @@ class LoopEntry(Part):
             raise ValueError(f"pass {number} of {self.times}")
         if isinstance(pending, (NormedAhead, K.RowSquares)):
             pending = None                         # the stream is complete already
+        elif pending is not None and pending.dtype != torch.float32:
+            pending = K.sum_parts(pending, None, torch.float32)
         both = K.concat_rows(x, x0, self.rt.dtype, delta=pending, write_back=False)
         out = K.sum_parts(self.mix.product(both, f32_ok=True), None if self.steps is None else self.steps[number], torch.float32)
         return out, None

@@ -692,6 +692,9 @@ def test_the_loops_entry_without_vectors(dtype):
             out, left = part.forward(None, _f32(x), None if delta is None else _f32(delta), _f32(x0), number)
             assert left is None and out.dtype == torch.float32
             _close(_np(out), np.concatenate([full, x0], axis=1) @ w["in"].T, 2 * PART_TOL[dtype])
+        half = _f32(d).bfloat16()                              # what the stream still lacks may come in the matrices' type
+        out, _ = part.forward(None, _f32(x), half, _f32(x0), number)
+        _close(_np(out), np.concatenate([x + _np(half), x0], axis=1) @ w["in"].T, 2 * PART_TOL[dtype])
 
 
 # ---------------------------------------------------------------------------
