@@ -407,7 +407,8 @@ __global__ void qk_rope_cache_kernel(const TI* __restrict__ qkv, int parts, size
 }
 
 // The same for head_dim = 128, rotated whole in split halves or (NEAR) the first `rot` dimensions, a
-// multiple of 4, in neighbouring pairs, without LDS or block barriers, for prompts.  With one (token, head) a wave and two values a lane this kernel took 29.5 us for 2,048
+// multiple of 4, in neighbouring pairs, without LDS or block barriers, for prompts.
+// With one (token, head) a wave and two values a lane this kernel took 29.5 us for 2,048
 // tokens of the 8B head shape (2.6 TB/s) and 20 us of that with every store left out: its time
 // was the number of its load instructions (five a token and head, of 4 and 8 bytes a lane), not
 // bytes or latency.  So a lane takes four consecutive dimensions (one 16-byte load), half a
